@@ -14,6 +14,7 @@ The reference plans its pools from per-class specs in the same spirit
 
 from __future__ import annotations
 
+import dataclasses
 from dataclasses import dataclass
 
 import torch
@@ -78,6 +79,13 @@ class CacheKind:
         can a new request take over pages that already hold its beginning (the prefix cache)."""
         return False
 
+    def joined(self, need, reader):
+        """The need of a memory that a run with need ``reader`` reads as well: what ``need`` holds, kept for as long as
+        either can still see it.  ``ValueError`` where the reader cannot use such a memory."""
+        if need != reader:
+            raise ValueError(f"{reader} differs from {need}")
+        return need
+
     def page_bytes(self, need, page_size: int, dtype: torch.dtype) -> int:
         return 0
 
@@ -98,8 +106,19 @@ class CacheKind:
         whose requests start in the coming step."""
 
 
+def _joined_window(need, reader):
+    """``need`` with the wider of the two windows; the rows themselves must be alike."""
+    if dataclasses.replace(reader, window=need.window) != need:
+        raise ValueError(f"{reader} differs from {need}")
+    both = need.window is not None and reader.window is not None
+    return dataclasses.replace(need, window=max(need.window, reader.window) if both else None)
+
+
 class PagedKeysValues(CacheKind):
     paged = True
+
+    def joined(self, need, reader):
+        return _joined_window(need, reader)
 
     def window(self, need):
         return need.window
@@ -127,6 +146,9 @@ class PagedLatents(CacheKind):
     """One row per token in pages, addressed through the same block tables as keys and values."""
 
     paged = True
+
+    def joined(self, need, reader):
+        return _joined_window(need, reader)
 
     def window(self, need):
         return need.window

@@ -37,11 +37,11 @@ def group_runs(model) -> tuple[list[int | None], list[int | None]]:
 
 def group_horizons(model) -> tuple[list[tuple], list[int | None]]:
     """((window, chunk) of each group, group of each run).  Runs whose mixers keep pages with the same
-    window and chunk share a group, that is, block tables."""
+    window and chunk share a group, that is, block tables; a run that reads another's pages is in that run's group,
+    whose window covers them both."""
     windows: list[tuple] = []
     run_group: list[int | None] = []
-    for run in model.order:
-        need = model.blocks[run.layer].mixer.cache_need()
+    for need in model.memory_needs():
         kind = kind_of(need)
         if kind is not None and kind.is_paged(need):
             window = (kind.window(need), kind.chunk(need))
@@ -60,11 +60,10 @@ def plan_cache(model, page_size: int, dtype: torch.dtype, *, num_pages: int | No
     windows, run_group = group_horizons(model)
     per_page = [0] * len(windows)
     per_slot = 0
-    for run, group in zip(model.order, run_group):
+    for run, group, need in zip(model.order, run_group, model.memory_needs()):
         if run.reads_run is not None:
             continue
         mixer = model.blocks[run.layer].mixer
-        need = mixer.cache_need()
         kind = kind_of(need)
         if kind is None:
             continue
@@ -111,8 +110,7 @@ class CacheStorage:
         self.device = torch.device(device)
         self.bindings: list = []
         self._owned: list[tuple] = []    # (kind, binding) of every run that owns memory
-        for i, (run, group) in enumerate(zip(model.order, plan.run_group)):
-            need = model.blocks[run.layer].mixer.cache_need()
+        for i, (run, group, need) in enumerate(zip(model.order, plan.run_group, model.memory_needs())):
             kind = kind_of(need)
             if kind is None:
                 self.bindings.append(None)

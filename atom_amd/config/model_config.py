@@ -689,6 +689,115 @@ class SavidraConfig(ModelConfig):
         return out
 
 
+@dataclass(frozen=True)
+class BenolixConfig(ModelConfig):
+    """``Benolix``: scaled token rows start a float32 stream that is normed after every sum, ``x <- norm(alpha x +
+    sublayer(x))``; layers are listed one by one, each attention over cached latents (queries through a latent of their
+    own, a window, a gate per output entry), with latents of its own or those of an earlier layer (``mixer.kv_from``),
+    and an optional feed-forward, dense or routed experts with softmax scores, some of them identities.  config.json keys:
+    ``vocab``, ``width``, ``embedding.scale``, ``norm.eps``, ``postln_alpha``, ``layers`` (``type``, ``mixer``,
+    ``mlp``)."""
+
+    layers: tuple = ()
+    norm_eps: float = 1e-6
+    embedding_scale: float = 1.0
+    postln_alpha: float = 1.0
+
+    model_type: ClassVar[str] = "benolix"
+    MIXER_TYPES: ClassVar[tuple] = ("latent_attention",)
+    MLP_KINDS: ClassVar[tuple] = ("dense", "moe")
+
+    @classmethod
+    def from_dict(cls, raw: dict) -> "BenolixConfig":
+        layers = _need(raw, "layers", list, "the model")
+        cfg = cls(
+            architecture=raw.get("architecture") or (raw.get("architectures") or ["Benolix"])[0],
+            vocab_size=_need(raw, "vocab", int, "the model"),
+            hidden_size=_need(raw, "width", int, "the model"),
+            num_hidden_layers=len(layers),
+            max_position_embeddings=_take(raw, "max_position_embeddings", int, 1 << 20),
+            tie_word_embeddings=False,
+            torch_dtype=str(raw.get("torch_dtype") or raw.get("dtype") or "bfloat16"),
+            bos_token_id=raw.get("bos_token_id"),
+            eos_token_id=raw.get("eos_token_id"),
+            layers=tuple(layers),
+            norm_eps=_need(raw.get("norm"), "eps", float, "'norm'"),
+            embedding_scale=_take(raw.get("embedding") or {}, "scale", float, 1.0),
+            postln_alpha=_take(raw, "postln_alpha", float, 1.0),
+        )
+        cfg.validate()
+        return cfg
+
+    def validate(self) -> None:
+        if self.vocab_size <= 0 or self.hidden_size <= 0 or not self.layers:
+            raise ConfigError("vocab, width and the number of layers must be positive")
+        if self.norm_eps <= 0:
+            raise ConfigError("norm.eps must be positive")
+
+        def positive(m, keys, where):
+            for key in keys:
+                if _need(m, key, int, where) <= 0:
+                    raise ConfigError(f"{where}: {key} must be positive")
+
+        for i, layer in enumerate(self.layers):
+            where = f"layer {i}"
+            kind = _need(layer, "type", str, where)
+            if kind not in self.MIXER_TYPES:
+                raise ConfigError(f"{where}: unknown type {kind!r}; known: {self.MIXER_TYPES}")
+            m = _need(layer, "mixer", dict, where)
+            mw = f"{where}'s mixer"
+            positive(m, ("heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank"), mw)
+            _need(m, "scale", float, mw)
+            rot = _need(m, "rot", dict, mw)
+            dims = _need(rot, "dims", int, f"{where}'s rot")
+            _need(rot, "base", float, f"{where}'s rot")
+            if dims % 2 or dims < 0 or dims > m["rot_dim"]:
+                raise ConfigError(f"{where}: rot.dims must be even and at most rot_dim")
+            if m.get("mask") is not None:
+                positive(m["mask"], ("size",), f"{where}'s mask")
+            if m.get("kv_from") is not None:
+                source = _need(m, "kv_from", int, mw)
+                if not 0 <= source < i:
+                    raise ConfigError(f"{where}: kv_from must name an earlier layer, got {source}")
+                theirs = self.layers[source]["mixer"]
+                if theirs.get("kv_from") is not None:
+                    raise ConfigError(f"{where}: kv_from names layer {source}, which has no latents of its own")
+                for key in ("kv_rank", "rot_dim", "rot"):
+                    if theirs[key] != m[key]:
+                        raise ConfigError(f"{where}: {key} must equal that of layer {source}, whose latents it reads")
+            mlp = layer.get("mlp")
+            if mlp is not None:
+                mk = _need(mlp, "kind", str, f"{where}'s mlp")
+                if mk not in self.MLP_KINDS:
+                    raise ConfigError(f"{where}: unknown mlp kind {mk!r}; known: {self.MLP_KINDS}")
+                if mk == "dense":
+                    positive(mlp, ("ff",), f"{where}'s mlp")
+                    continue
+                expert = _need(mlp, "expert", dict, f"{where}'s mlp")
+                positive(expert, ("ff",), f"{where}'s mlp.expert")
+                if _need(expert, "limit", float, f"{where}'s mlp.expert") <= 0:
+                    raise ConfigError(f"{where}: expert.limit must be positive")
+                router = _need(mlp, "router", dict, f"{where}'s mlp")
+                positive(router, ("experts", "top"), f"{where}'s router")
+                identity = _take(router, "identity", int, 0)
+                _take(router, "scale", float, 1.0)
+                if identity < 0 or router["top"] > router["experts"] + identity:
+                    raise ConfigError(f"{where}: the router's top must lie in 1 .. experts + identity")
+
+    def to_dict(self) -> dict:
+        out: dict[str, Any] = {
+            "architecture": self.architecture, "model_type": self.model_type, "vocab": self.vocab_size,
+            "width": self.hidden_size, "embedding": {"scale": self.embedding_scale}, "norm": {"eps": self.norm_eps},
+            "postln_alpha": self.postln_alpha, "layers": [dict(layer) for layer in self.layers],
+        }
+        if self.max_position_embeddings != 1 << 20:
+            out["max_position_embeddings"] = self.max_position_embeddings
+        for key in ("bos_token_id", "eos_token_id"):
+            if getattr(self, key) is not None:
+                out[key] = getattr(self, key)
+        return out
+
+
 def read_config_json(folder: str) -> dict:
     path = os.path.join(folder, "config.json")
     if not os.path.isfile(path):

@@ -7,8 +7,8 @@ from __future__ import annotations
 from dataclasses import dataclass
 from typing import Callable
 
-from .model_config import (ConfigError, LeduvikConfig, LotoraxConfig, ModelConfig, Qwen3Config, RalitarConfig,
-                           SavidraConfig)
+from .model_config import (BenolixConfig, ConfigError, LeduvikConfig, LotoraxConfig, ModelConfig, Qwen3Config,
+                           RalitarConfig, SavidraConfig)
 
 
 @dataclass(frozen=True)
@@ -88,3 +88,7 @@ def _ensure_builtin() -> None:
 
     if "Savidra" not in _ARCHITECTURES:
         register_architecture("Savidra", SavidraConfig, savidra_spec)
+    from ..models.benolix import benolix_spec
+
+    if "Benolix" not in _ARCHITECTURES:
+        register_architecture("Benolix", BenolixConfig, benolix_spec)

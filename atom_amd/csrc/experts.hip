@@ -1,24 +1,44 @@
 // A feed-forward of routed experts: every token is sent to `top` of `experts` small gated feed-forwards and
 // receives the weighted sum of their outputs.
 //
-//   router_choose     from float32 router logits z: s = sigmoid(z); the `top` experts with the largest s + correction
-//                     are chosen (ties: the lower index); a chosen expert's weight is its s, or s divided by the
-//                     chosen experts' sum when `renormalize` is set
-//   experts_gate_up   for every (token, choice): act = f(W_gate[e] x) * (W_up[e] x), W stored [experts, 2 ff, width]
+//   router_choose     from float32 router logits z: s = sigmoid(z), or s = softmax(z) over all of a token's logits; the
+//                     `top` experts with the largest s + correction are chosen (ties: the lower index); a chosen
+//                     expert's weight is its s, or s divided by (the chosen experts' sum + eps) when `renormalize` is
+//                     set, times `scale`
+//   experts_gate_up   for every (token, choice): act = f(W_gate[e] x, W_up[e] x), W stored [experts, 2 ff, width]
 //   experts_down      y[t] = sum over the token's choices, in their order, of weight * W_down[e] act
+//
+// A router may have more outputs than there are experts: the outputs from `experts` on are identity experts, whose
+// result is x itself (no matrices); the down and combine kernels add weight * x for them.
+//
+// f(g, u) is act(g) * u, or for SiLU more generally, with g' = min(g, limit) and u' = u clamped to [-limit, limit],
+// g' * sigmoid(slope * g') * (u' + shift); limit = infinity, slope 1 and shift 0 are the plain SiLU gate.
 //
 // The last two read an expert's rows once per (token, choice): the form for steps of few tokens.  Every sum runs in a
 // fixed order over a token's own data, so a token's result does not depend on what else is in the batch.
 #include "common.h"
 
+struct RouterRule {
+  int softmax;        // scores: 0 sigmoid, 1 softmax over the token's logits
+  int renormalize;
+  float eps, scale;   // weight = s / (sum of the chosen + eps) * scale, or s * scale
+};
+
 __global__ void router_choose_kernel(const float* __restrict__ logits, const float* __restrict__ correction,
                                      int* __restrict__ ids, float* __restrict__ weights, int tokens, int experts,
-                                     int top, int renormalize) {
+                                     int top, RouterRule rule) {
   const int t = blockIdx.x * blockDim.x + threadIdx.x;
   if (t >= tokens) return;
   const float* z = logits + (size_t)t * experts;
   int* mine = ids + (size_t)t * top;
   float* w = weights + (size_t)t * top;
+  float peak = 0.f, denom = 1.f;
+  if (rule.softmax) {
+    peak = -INFINITY;
+    for (int e = 0; e < experts; ++e) peak = fmaxf(peak, z[e]);
+    denom = 0.f;
+    for (int e = 0; e < experts; ++e) denom += expf(z[e] - peak);
+  }
   float total = 0.f;
   for (int k = 0; k < top; ++k) {
     int best = -1;
@@ -27,7 +47,7 @@ __global__ void router_choose_kernel(const float* __restrict__ logits, const flo
       bool taken = false;
       for (int j = 0; j < k; ++j) taken |= (mine[j] == e);
       if (taken) continue;
-      const float s = 1.f / (1.f + expf(-z[e]));
+      const float s = rule.softmax ? expf(z[e] - peak) / denom : 1.f / (1.f + expf(-z[e]));
       const float score = s + (correction ? correction[e] : 0.f);
       if (best < 0 || score > best_score) {
         best = e;
@@ -39,8 +59,7 @@ __global__ void router_choose_kernel(const float* __restrict__ logits, const flo
     w[k] = best_s;
     total += best_s;
   }
-  if (renormalize)
-    for (int k = 0; k < top; ++k) w[k] /= total;
+  for (int k = 0; k < top; ++k) w[k] = (rule.renormalize ? w[k] / (total + rule.eps) : w[k]) * rule.scale;
 }
 
 // A wave per token: lane l holds the scores of experts l, l + 64, ... (up to 8 of them, so up to 512 experts); each
@@ -50,16 +69,32 @@ constexpr int kRouterPerLane = 8;
 __global__ void __launch_bounds__(256)
 router_choose_wave_kernel(const float* __restrict__ logits, const float* __restrict__ correction,
                           int* __restrict__ ids, float* __restrict__ weights, int tokens, int experts, int top,
-                          int renormalize) {
+                          RouterRule rule) {
   const int t = blockIdx.x * 4 + threadIdx.x / kWave;
   if (t >= tokens) return;
   const int lane = threadIdx.x % kWave;
   float score[kRouterPerLane], plain[kRouterPerLane];
+  float peak = -INFINITY, denom = 0.f;
+#pragma unroll
+  for (int j = 0; j < kRouterPerLane; ++j) {
+    const int e = lane + j * kWave;
+    plain[j] = e < experts ? logits[(size_t)t * experts + e] : -INFINITY;
+    peak = fmaxf(peak, plain[j]);
+  }
+  if (rule.softmax) {
+    peak = wave_max(peak);
+#pragma unroll
+    for (int j = 0; j < kRouterPerLane; ++j) {
+      plain[j] = expf(plain[j] - peak);
+      denom += plain[j];
+    }
+    denom = wave_sum(denom);
+  }
 #pragma unroll
   for (int j = 0; j < kRouterPerLane; ++j) {
     const int e = lane + j * kWave;
     if (e < experts) {
-      plain[j] = 1.f / (1.f + expf(-logits[(size_t)t * experts + e]));
+      plain[j] = rule.softmax ? plain[j] / denom : 1.f / (1.f + expf(-plain[j]));
       score[j] = plain[j] + (correction ? correction[e] : 0.f);
     } else {
       plain[j] = 0.f;
@@ -90,33 +125,45 @@ router_choose_wave_kernel(const float* __restrict__ logits, const float* __restr
 #pragma unroll
     for (int j = 0; j < kRouterPerLane; ++j)
       if (lane + j * kWave == best_e) score[j] = -INFINITY;
+    if (best_e >= experts) best_e = k;   // scores that are no numbers: an index the next kernels can follow all the same
     if (lane == 0) ids[(size_t)t * top + k] = best_e;
     if (lane == k) mine = best_plain;
     total += best_plain;
   }
-  if (lane < top) weights[(size_t)t * top + lane] = renormalize ? mine / total : mine;
+  if (lane < top) weights[(size_t)t * top + lane] = (rule.renormalize ? mine / (total + rule.eps) : mine) * rule.scale;
 }
 
 ATOM_EXPORT int atom_router_choose(const float* logits, const float* correction, int* ids, float* weights, int tokens,
-                                   int experts, int top, int renormalize, hipStream_t stream) {
+                                   int experts, int top, int softmax, int renormalize, float eps, float scale,
+                                   hipStream_t stream) {
   if (tokens < 0 || experts <= 0 || top <= 0 || top > experts) return ATOM_BAD_SHAPE;
   if (logits == nullptr || ids == nullptr || weights == nullptr) return ATOM_BAD_SHAPE;
   if (tokens == 0) return ATOM_OK;
+  const RouterRule rule{softmax, renormalize, eps, scale};
   if (experts <= kRouterPerLane * kWave && top <= kWave) {
     hipLaunchKernelGGL(router_choose_wave_kernel, dim3((tokens + 3) / 4), dim3(256), 0, stream, logits, correction, ids,
-                       weights, tokens, experts, top, renormalize);
+                       weights, tokens, experts, top, rule);
     return launch_status();
   }
   hipLaunchKernelGGL(router_choose_kernel, dim3((tokens + 127) / 128), dim3(128), 0, stream, logits, correction, ids,
-                     weights, tokens, experts, top, renormalize);
+                     weights, tokens, experts, top, rule);
   return launch_status();
 }
 
-__device__ __forceinline__ float expert_activation(float g, int act) {
-  if (act == 1) return g > 0.f ? g : 0.f;
-  if (act == 2) return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
-  return g / (1.f + expf(-g));
+struct ExpertGate {
+  int act;                     // 0 SiLU, 1 ReLU, 2 tanh-GELU
+  float limit, slope, shift;   // SiLU only
+};
+
+__device__ __forceinline__ float expert_gate(float g, float u, const ExpertGate& f) {
+  if (f.act == 1) return (g > 0.f ? g : 0.f) * u;
+  if (f.act == 2) return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
+  g = fminf(g, f.limit);
+  u = fminf(fmaxf(u, -f.limit), f.limit);
+  return g / (1.f + expf(-f.slope * g)) * (u + f.shift);
 }
+
+static bool expert_gate_ok(const ExpertGate& f) { return f.act >= 0 && f.act <= 2 && f.limit > 0.f; }
 
 constexpr int kExpCols = 32;   // output columns of a block: 4 waves x 8
 typedef __attribute__((ext_vector_type(8))) __bf16 ex_bf16x8;
@@ -124,11 +171,12 @@ typedef __attribute__((ext_vector_type(8))) __bf16 ex_bf16x8;
 template <typename T, typename TW>
 __global__ void __launch_bounds__(256)
 experts_gate_up_kernel(const T* __restrict__ x, const TW* __restrict__ w, const int* __restrict__ ids,
-                       T* __restrict__ act_out, int top, int ff, int width, int act) {
+                       T* __restrict__ act_out, int top, int experts, int ff, int width, ExpertGate f) {
   extern __shared__ float xs[];   // width
   const int pair = blockIdx.x;
   const int t = pair / top;
   const int e = ids[pair];
+  if (e >= experts) return;       // an identity expert: the down kernel adds x itself
   const int tid = threadIdx.x, wave = tid / kWave, lane = tid % kWave;
   const T* xr = x + (size_t)t * width;
   for (int i = tid; i < width; i += 256) xs[i] = to_f32(xr[i]);
@@ -165,14 +213,15 @@ experts_gate_up_kernel(const T* __restrict__ x, const TW* __restrict__ w, const 
     }
     g = wave_sum(g);
     u = wave_sum(u);
-    if (lane == 0) act_out[(size_t)pair * ff + col] = from_f32<T>(expert_activation(g, act) * u);
+    if (lane == 0) act_out[(size_t)pair * ff + col] = from_f32<T>(expert_gate(g, u, f));
   }
 }
 
 template <typename T, typename TW>
 __global__ void __launch_bounds__(256)
-experts_down_kernel(const T* __restrict__ act_in, const TW* __restrict__ w, const int* __restrict__ ids,
-                    const float* __restrict__ weights, T* __restrict__ y, int top, int ff, int width) {
+experts_down_kernel(const T* __restrict__ x, const T* __restrict__ act_in, const TW* __restrict__ w,
+                    const int* __restrict__ ids, const float* __restrict__ weights, T* __restrict__ y, int top, int experts,
+                    int ff, int width) {
   extern __shared__ float as[];   // top * ff
   const int t = blockIdx.x;
   const int tid = threadIdx.x, wave = tid / kWave, lane = tid % kWave;
@@ -184,6 +233,10 @@ experts_down_kernel(const T* __restrict__ act_in, const TW* __restrict__ w, cons
     float total = 0.f;
     for (int k = 0; k < top; ++k) {
       const int e = ids[(size_t)t * top + k];
+      if (e >= experts) {
+        total += weights[(size_t)t * top + k] * to_f32(x[(size_t)t * width + col]);
+        continue;
+      }
       const TW* wr = w + ((size_t)e * width + col) * ff;
       float s = 0.f;
       bool done = false;
@@ -206,8 +259,10 @@ experts_down_kernel(const T* __restrict__ act_in, const TW* __restrict__ w, cons
 }
 
 ATOM_EXPORT int atom_experts_gate_up(const void* x, const void* w, int w_dtype, const int* ids, void* act_out, int dtype,
-                                     int tokens, int top, int ff, int width, int act, hipStream_t stream) {
-  if (tokens < 0 || top <= 0 || ff <= 0 || width <= 0 || act < 0 || act > 2) return ATOM_BAD_SHAPE;
+                                     int tokens, int top, int experts, int ff, int width, int act, float limit, float slope,
+                                     float shift, hipStream_t stream) {
+  const ExpertGate f{act, limit, slope, shift};
+  if (tokens < 0 || top <= 0 || experts <= 0 || ff <= 0 || width <= 0 || !expert_gate_ok(f)) return ATOM_BAD_SHAPE;
   if (x == nullptr || w == nullptr || ids == nullptr || act_out == nullptr) return ATOM_BAD_SHAPE;
   if ((size_t)width * sizeof(float) > 64 * 1024) return ATOM_TOO_LARGE;
   if (tokens == 0) return ATOM_OK;
@@ -216,7 +271,7 @@ ATOM_EXPORT int atom_experts_gate_up(const void* x, const void* w, int w_dtype, 
   const size_t smem = (size_t)width * sizeof(float);
 #define LAUNCH(T, TW)                                                                                              \
   hipLaunchKernelGGL((experts_gate_up_kernel<T, TW>), grid, block, smem, stream, (const T*)x, (const TW*)w, ids, \
-                     (T*)act_out, top, ff, width, act)
+                     (T*)act_out, top, experts, ff, width, f)
   if (dtype == ATOM_F32 && w_dtype == ATOM_F32) LAUNCH(float, float);
   else if (dtype == ATOM_BF16 && w_dtype == ATOM_BF16) LAUNCH(bf16_t, bf16_t);
   else if (dtype == ATOM_BF16 && w_dtype == ATOM_F32) LAUNCH(bf16_t, float);
@@ -225,18 +280,19 @@ ATOM_EXPORT int atom_experts_gate_up(const void* x, const void* w, int w_dtype, 
   return launch_status();
 }
 
-ATOM_EXPORT int atom_experts_down(const void* act_in, const void* w, int w_dtype, const int* ids, const float* weights,
-                                  void* y, int dtype, int tokens, int top, int ff, int width, hipStream_t stream) {
-  if (tokens < 0 || top <= 0 || ff <= 0 || width <= 0) return ATOM_BAD_SHAPE;
-  if (act_in == nullptr || w == nullptr || ids == nullptr || weights == nullptr || y == nullptr) return ATOM_BAD_SHAPE;
+ATOM_EXPORT int atom_experts_down(const void* x, const void* act_in, const void* w, int w_dtype, const int* ids,
+                                  const float* weights, void* y, int dtype, int tokens, int top, int experts, int ff,
+                                  int width, hipStream_t stream) {
+  if (tokens < 0 || top <= 0 || experts <= 0 || ff <= 0 || width <= 0) return ATOM_BAD_SHAPE;
+  if (x == nullptr || act_in == nullptr || w == nullptr || ids == nullptr || weights == nullptr || y == nullptr) return ATOM_BAD_SHAPE;
   if ((size_t)top * ff * sizeof(float) > 64 * 1024) return ATOM_TOO_LARGE;
   if (tokens == 0) return ATOM_OK;
   dim3 grid(tokens, (width + kExpCols - 1) / kExpCols), block(256);
   if (grid.y > 65535) return ATOM_TOO_LARGE;
   const size_t smem = (size_t)top * ff * sizeof(float);
 #define LAUNCH(T, TW)                                                                                               \
-  hipLaunchKernelGGL((experts_down_kernel<T, TW>), grid, block, smem, stream, (const T*)act_in, (const TW*)w, ids, \
-                     weights, (T*)y, top, ff, width)
+  hipLaunchKernelGGL((experts_down_kernel<T, TW>), grid, block, smem, stream, (const T*)x, (const T*)act_in,       \
+                     (const TW*)w, ids, weights, (T*)y, top, experts, ff, width)
   if (dtype == ATOM_F32 && w_dtype == ATOM_F32) LAUNCH(float, float);
   else if (dtype == ATOM_BF16 && w_dtype == ATOM_BF16) LAUNCH(bf16_t, bf16_t);
   else if (dtype == ATOM_BF16 && w_dtype == ATOM_F32) LAUNCH(bf16_t, float);
@@ -249,13 +305,13 @@ ATOM_EXPORT int atom_experts_down(const void* act_in, const void* w, int w_dtype
 //
 //   experts_sort      one block: counts the pairs of every expert, gives each expert whole tiles of 64 rows
 //                     (padded), and every pair its row.  tile_expert[tile] = expert or -1; row_pair[row] = pair or
-//                     -1; pair_row[pair] = row.  Rows of one expert come in no fixed order; a row's result does
-//                     not depend on its place.
-//   grouped_gate_up   act[row] = f(W_gate[e] x) * (W_up[e] x) for the rows of a tile, on the matrix cores.  The
+//                     -1; pair_row[pair] = row, or -1 for an identity expert's pair, which gets none.  Rows of one
+//                     expert come in no fixed order; a row's result does not depend on its place.
+//   grouped_gate_up   act[row] = f(W_gate[e] x, W_up[e] x) for the rows of a tile, on the matrix cores.  The
 //                     weights are the A operand and the tokens the B operand, both read straight from memory in
 //                     16-byte pieces, so a lane ends up with four consecutive columns of one row.
 //   grouped_down      y[row] = W_down[e] act[row], float32
-//   experts_combine   out[t] = sum_k weight[t, k] * y[pair_row[t, k]], in the order of k
+//   experts_combine   out[t] = sum_k weight[t, k] * (y[pair_row[t, k]], or x[t] where that is -1), in the order of k
 //
 // bfloat16 only; width and ff multiples of 8.
 
@@ -276,7 +332,8 @@ experts_sort_kernel(const int* __restrict__ ids, int pairs, int experts, int max
   for (int i = tid; i < max_tiles; i += 1024) tile_expert[i] = -1;
   for (int i = tid; i < max_tiles * kTileRows; i += 1024) row_pair[i] = -1;
   __syncthreads();
-  for (int i = tid; i < pairs; i += 1024) atomicAdd(&counts[ids[i]], 1);
+  for (int i = tid; i < pairs; i += 1024)
+    if (ids[i] < experts) atomicAdd(&counts[ids[i]], 1);
   __syncthreads();
   if (tid == 0) {
     int tile = 0;
@@ -291,6 +348,10 @@ experts_sort_kernel(const int* __restrict__ ids, int pairs, int experts, int max
   __syncthreads();
   for (int i = tid; i < pairs; i += 1024) {
     const int e = ids[i];
+    if (e >= experts) {
+      pair_row[i] = -1;
+      continue;
+    }
     const int row = first[e] + atomicAdd(&counts[e], 1);
     row_pair[row] = i;
     pair_row[i] = row;
@@ -306,7 +367,7 @@ __device__ __forceinline__ bf16x8 load8(const bf16_t* p, bool ok) {
 __global__ void __launch_bounds__(256)
 grouped_gate_up_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, const int* __restrict__ tile_expert,
                        const int* __restrict__ row_pair, bf16_t* __restrict__ act_out, int top, int ff, int width,
-                       int act) {
+                       ExpertGate f) {
   const int tile = blockIdx.x;
   const int e = tile_expert[tile];
   if (e < 0) return;
@@ -366,12 +427,12 @@ grouped_gate_up_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ 
       if (col + 3 < ff) {
         bf16x4 o;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) o[i] = static_cast<__bf16>(expert_activation(ga[ct][rt][i], act) * ua[ct][rt][i]);
+        for (int i = 0; i < 4; ++i) o[i] = static_cast<__bf16>(expert_gate(ga[ct][rt][i], ua[ct][rt][i], f));
         *reinterpret_cast<bf16x4*>(act_out + (size_t)row * ff + col) = o;
       } else {
         for (int i = 0; i < 4; ++i)
           if (col + i < ff)
-            act_out[(size_t)row * ff + col + i] = static_cast<bf16_t>(expert_activation(ga[ct][rt][i], act) * ua[ct][rt][i]);
+            act_out[(size_t)row * ff + col + i] = static_cast<bf16_t>(expert_gate(ga[ct][rt][i], ua[ct][rt][i], f));
       }
     }
   }
@@ -433,12 +494,16 @@ grouped_down_kernel(const bf16_t* __restrict__ act_in, const bf16_t* __restrict_
   }
 }
 
-__global__ void experts_combine_kernel(const float* __restrict__ y, const int* __restrict__ pair_row,
-                                       const float* __restrict__ weights, bf16_t* __restrict__ out, int top, int width) {
+__global__ void experts_combine_kernel(const float* __restrict__ y, const bf16_t* __restrict__ x,
+                                       const int* __restrict__ pair_row, const float* __restrict__ weights,
+                                       bf16_t* __restrict__ out, int top, int width) {
   const size_t t = blockIdx.x;
   for (int c = threadIdx.x; c < width; c += blockDim.x) {
     float total = 0.f;
-    for (int k = 0; k < top; ++k) total += weights[t * top + k] * y[(size_t)pair_row[t * top + k] * width + c];
+    for (int k = 0; k < top; ++k) {
+      const int row = pair_row[t * top + k];
+      total += weights[t * top + k] * (row >= 0 ? y[(size_t)row * width + c] : to_f32(x[t * width + c]));
+    }
     out[t * width + c] = static_cast<bf16_t>(total);
   }
 }
@@ -456,8 +521,9 @@ ATOM_EXPORT int atom_experts_grouped_supports(int ff, int width, int experts) {
 ATOM_EXPORT int atom_experts_grouped(const void* x, const void* gate_up, const void* down, const int* ids,
                                      const float* weights, int* tile_expert, int* row_pair, int* pair_row, void* act_buf,
                                      float* y, void* out, int tokens, int top, int experts, int ff, int width, int act,
-                                     hipStream_t stream) {
-  if (tokens < 0 || top <= 0 || act < 0 || act > 2) return ATOM_BAD_SHAPE;
+                                     float limit, float slope, float shift, hipStream_t stream) {
+  const ExpertGate f{act, limit, slope, shift};
+  if (tokens < 0 || top <= 0 || !expert_gate_ok(f)) return ATOM_BAD_SHAPE;
   if (!atom_experts_grouped_supports(ff, width, experts)) return ATOM_UNSUPPORTED;
   if (tokens == 0) return ATOM_OK;
   const int pairs = tokens * top;
@@ -466,10 +532,10 @@ ATOM_EXPORT int atom_experts_grouped(const void* x, const void* gate_up, const v
   hipLaunchKernelGGL(experts_sort_kernel, dim3(1), dim3(1024), 2 * experts * sizeof(int), stream, ids, pairs, experts,
                      tiles, tile_expert, row_pair, pair_row);
   hipLaunchKernelGGL(grouped_gate_up_kernel, dim3(tiles, (ff + 63) / 64), dim3(256), 0, stream, (const bf16_t*)x,
-                     (const bf16_t*)gate_up, tile_expert, row_pair, (bf16_t*)act_buf, top, ff, width, act);
+                     (const bf16_t*)gate_up, tile_expert, row_pair, (bf16_t*)act_buf, top, ff, width, f);
   hipLaunchKernelGGL(grouped_down_kernel, dim3(tiles, (width + 127) / 128), dim3(256), 0, stream, (const bf16_t*)act_buf,
                      (const bf16_t*)down, tile_expert, y, ff, width);
-  hipLaunchKernelGGL(experts_combine_kernel, dim3(tokens), dim3(256), 0, stream, y, pair_row, weights, (bf16_t*)out, top,
-                     width);
+  hipLaunchKernelGGL(experts_combine_kernel, dim3(tokens), dim3(256), 0, stream, y, (const bf16_t*)x, pair_row, weights,
+                     (bf16_t*)out, top, width);
   return launch_status();
 }

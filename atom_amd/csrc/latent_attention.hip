@@ -7,9 +7,10 @@
 //   o_lat[t, h]    = sum_j softmax_j(score)[j] * c[j],   the softmax's denominator holding exp(sink[h]) as well
 //
 // Pages: [num_pages, page_size, rank + rot].  Three kernels:
-//   latent_prepare      norms the new latents, rotates the new keys' shared part and writes both to their pages;
-//                       rotates the queries' rotated parts into q_abs[.., rank:]
-//   heads_gemm          y[t, h, :] = alpha * x[t, h, :] W_h^T (* sigmoid(gate[t, h])), one small product per head
+//   latent_prepare      norms the new latents, rotates the new keys' shared part and writes both to their pages; norms
+//                       the latent that queries are projected up from, where a design has one
+//   heads_gemm          y[t, h, :] = alpha * x[t, h, :] W_h^T (* sigmoid(gate)), one small product per head; the
+//                       absorbing product takes the rotation of the queries' rotated parts with it (QueryTurn)
 //   latent_attention    scores, softmax with sink, weighted sum; any sizes, float32 or bfloat16 pages
 //
 // Rotation: entries (2i, 2i + 1) of the rotated part are a pair; its angle is position * freq[i], formed in
@@ -27,21 +28,31 @@ __device__ __forceinline__ void pair_angle(int position, double freq, float mult
   *s = sf * mult;
 }
 
-// proj [tokens, ld] float32: queries at q_off (H heads of dim + rot), then the down-projection at kv_off
-// (rank entries, then rot).
+// proj [tokens, ld] float32 holds, where asked for, the latent of the queries at cq_off (cq_rank entries) and the
+// down-projection of the keys at kv_off (rank entries, then rot).  A block a token.
 template <typename T>
 __global__ void __launch_bounds__(256)
-latent_prepare_kernel(const float* __restrict__ proj, int ld, int q_off, int kv_off, int heads, int dim, int rot,
-                      int rank, int rot_dims, const float* __restrict__ norm_w, float eps,
-                      const double* __restrict__ freq, float mult, const int* __restrict__ positions,
-                      const int* __restrict__ slots, T* __restrict__ pages, T* __restrict__ q_abs, float q_scale) {
+latent_prepare_kernel(const float* __restrict__ proj, int ld, int cq_off, int cq_rank, const float* __restrict__ cq_w,
+                      T* __restrict__ cq, int kv_off, int rank, int rot, int rot_dims, const float* __restrict__ norm_w,
+                      float eps, const double* __restrict__ freq, float mult, const int* __restrict__ positions,
+                      const int* __restrict__ slots, T* __restrict__ pages) {
   __shared__ float scratch[16];
   const int t = blockIdx.x;
   const int tid = threadIdx.x;
   const float* row = proj + (size_t)t * ld;
+  if (cq_rank > 0) {
+    float part = 0.f;
+    for (int i = tid; i < cq_rank; i += 256) {
+      const float v = row[cq_off + i];
+      part += v * v;
+    }
+    const float rstd = 1.f / sqrtf(block_sum(part, scratch) / (float)cq_rank + eps);
+    for (int i = tid; i < cq_rank; i += 256) cq[(size_t)t * cq_rank + i] = from_f32<T>(row[cq_off + i] * rstd * cq_w[i]);
+  }
+  const int slot = slots ? slots[t] : -1;   // the same for the whole block
+  if (slot < 0) return;
   const int pos = positions[t];
-  const int width = rank + rot;
-  const int slot = slots ? slots[t] : -1;
+  T* dst = pages + (size_t)slot * (rank + rot);
   // the latent: x / sqrt(mean(x^2) + eps) * w
   float part = 0.f;
   for (int i = tid; i < rank; i += 256) {
@@ -49,58 +60,88 @@ latent_prepare_kernel(const float* __restrict__ proj, int ld, int q_off, int kv_
     part += v * v;
   }
   const float rstd = 1.f / sqrtf(block_sum(part, scratch) / (float)rank + eps);
-  if (slot >= 0) {
-    T* dst = pages + (size_t)slot * width;
-    for (int i = tid; i < rank; i += 256) dst[i] = from_f32<T>(row[kv_off + i] * rstd * norm_w[i]);
-    // the shared rotated key part
-    for (int i = tid; i < rot; i += 256) {
-      float v = row[kv_off + rank + i];
-      if (i < rot_dims) {
-        float c, s;
-        pair_angle(pos, freq[i >> 1], mult, &c, &s);
-        const float other = row[kv_off + rank + (i ^ 1)];
-        v = (i & 1) ? v * c + other * s : v * c - other * s;
-      }
-      dst[rank + i] = from_f32<T>(v);
-    }
-  }
-  // the queries' rotated parts, scaled
-  const int per_head = dim + rot;
-  for (int idx = tid; idx < heads * rot; idx += 256) {
-    const int h = idx / rot, i = idx - h * rot;
-    const float* qr = row + q_off + h * per_head + dim;
-    float v = qr[i];
+  for (int i = tid; i < rank; i += 256) dst[i] = from_f32<T>(row[kv_off + i] * rstd * norm_w[i]);
+  // the shared rotated key part
+  for (int i = tid; i < rot; i += 256) {
+    float v = row[kv_off + rank + i];
     if (i < rot_dims) {
       float c, s;
       pair_angle(pos, freq[i >> 1], mult, &c, &s);
-      const float other = qr[i ^ 1];
+      const float other = row[kv_off + rank + (i ^ 1)];
       v = (i & 1) ? v * c + other * s : v * c - other * s;
     }
-    q_abs[((size_t)t * heads + h) * width + rank + i] = from_f32<T>(v * q_scale);
+    dst[rank + i] = from_f32<T>(v);
   }
 }
 
-ATOM_EXPORT int atom_latent_prepare(const float* proj, int ld, int q_off, int kv_off, int heads, int dim, int rot,
-                                    int rank, int rot_dims, const float* norm_w, float eps, const double* freq,
-                                    float mult, const int* positions, const int* slots, void* pages, void* q_abs,
-                                    int dtype, int tokens, float q_scale, hipStream_t stream) {
-  if (tokens < 0 || heads <= 0 || dim < 0 || rot < 0 || rank <= 0 || ld <= 0) return ATOM_BAD_SHAPE;
-  if (rot_dims < 0 || rot_dims > rot || (rot_dims & 1)) return ATOM_BAD_SHAPE;
-  if (q_off < 0 || kv_off < 0 || q_off + heads * (dim + rot) > ld || kv_off + rank + rot > ld) return ATOM_BAD_SHAPE;
-  if (proj == nullptr || norm_w == nullptr || positions == nullptr || q_abs == nullptr) return ATOM_BAD_SHAPE;
-  if (rot_dims > 0 && freq == nullptr) return ATOM_BAD_SHAPE;
-  if (slots != nullptr && pages == nullptr) return ATOM_BAD_SHAPE;
-  if (tokens == 0) return ATOM_OK;
+ATOM_EXPORT int atom_latent_prepare(const float* proj, int ld, int cq_off, int cq_rank, const float* cq_w, void* cq,
+                                    int kv_off, int rank, int rot, int rot_dims, const float* norm_w, float eps,
+                                    const double* freq, float mult, const int* positions, const int* slots, void* pages,
+                                    int dtype, int tokens, hipStream_t stream) {
+  if (tokens < 0 || ld <= 0 || cq_rank < 0 || proj == nullptr) return ATOM_BAD_SHAPE;
+  if (cq_rank > 0 && (cq_off < 0 || cq_off + cq_rank > ld || cq_w == nullptr || cq == nullptr)) return ATOM_BAD_SHAPE;
+  if (slots != nullptr) {
+    if (rot < 0 || rank <= 0 || rot_dims < 0 || rot_dims > rot || (rot_dims & 1)) return ATOM_BAD_SHAPE;
+    if (kv_off < 0 || kv_off + rank + rot > ld) return ATOM_BAD_SHAPE;
+    if (norm_w == nullptr || positions == nullptr || pages == nullptr) return ATOM_BAD_SHAPE;
+    if (rot_dims > 0 && freq == nullptr) return ATOM_BAD_SHAPE;
+  }
+  if (tokens == 0 || (cq_rank == 0 && slots == nullptr)) return ATOM_OK;
   ATOM_DISPATCH_DTYPE(dtype, hipLaunchKernelGGL((latent_prepare_kernel<T>), dim3(tokens), dim3(256), 0, stream, proj, ld,
-                                                 q_off, kv_off, heads, dim, rot, rank, rot_dims, norm_w, eps, freq, mult,
-                                                 positions, slots, (T*)pages, (T*)q_abs, q_scale));
+                                                 cq_off, cq_rank, cq_w, (T*)cq, kv_off, rank, rot, rot_dims, norm_w, eps,
+                                                 freq, mult, positions, slots, (T*)pages));
   return launch_status();
+}
+
+// The rotated parts of the queries, which go past the absorbing product: out[t, h, :] = scale * (x[t, h, :] with its
+// first rot_dims entries turned).  The product's launch has one more column of blocks for them.
+struct QueryTurn {
+  const float* x;        // [tokens, ..] float32: head h's rotated part at t * ldx + h * hsx
+  void* out;             // the product's output type: at t * ldo + h * hso
+  long ldx, hsx, ldo, hso;
+  const double* freq;
+  const int* positions;
+  int rot, rot_dims;     // rot 0: nothing to do
+  float mult, scale;
+};
+
+// Tokens t0 .. t0 + count - 1 of head h, by a block of 256 threads: an item is a pair of neighbours (or a last single).
+template <typename T>
+__device__ __forceinline__ void turn_queries(const QueryTurn& q, int h, int t0, int count) {
+  const int pairs = (q.rot + 1) / 2;
+  for (int idx = threadIdx.x; idx < count * pairs; idx += 256) {
+    const int t = t0 + idx / pairs, i = 2 * (idx % pairs);
+    const float* src = q.x + (size_t)t * q.ldx + (size_t)h * q.hsx + i;
+    T* dst = reinterpret_cast<T*>(q.out) + (size_t)t * q.ldo + (size_t)h * q.hso + i;
+    const bool both = i + 1 < q.rot;
+    float u = src[0], v = both ? src[1] : 0.f;
+    if (i < q.rot_dims) {
+      float c, s;
+      pair_angle(q.positions[t], q.freq[i >> 1], q.mult, &c, &s);
+      const float a = u * c - v * s;
+      v = v * c + u * s;
+      u = a;
+    }
+    dst[0] = from_f32<T>(u * q.scale);
+    if (both) dst[1] = from_f32<T>(v * q.scale);
+  }
+}
+
+// A gate on the product's output: y *= sigmoid(gate), one value per (token, head) or one per entry.
+struct ProductGate {
+  const float* g;       // null: none
+  long ldg;             // entry (t, h, c) at t * ldg + h * hsg + c * csg
+  int hsg, csg;
+};
+
+__device__ __forceinline__ float gate_value(const ProductGate& g, size_t t, int h, int c) {
+  return 1.f / (1.f + expf(-g.g[t * g.ldg + (size_t)h * g.hsg + (size_t)c * g.csg]));
 }
 
 // ------------------------------------------------------------------ one small product per head
 //
 // y[t * ldy + h * hsy + n] = alpha * sum_k x[t * ldx + h * hsx + k] * w[(h * N + n) * K + k]
-//                            (* sigmoid(gate[t * ldg + h]) when gate is given)
+//                            (* sigmoid of the gate when one is given)
 // float32 FMA in ascending k, 64 x 64 tiles, K walked 16 at a time through LDS.
 
 constexpr int kHTile = 64;
@@ -109,13 +150,17 @@ constexpr int kHStep = 16;
 template <typename TX, typename TW, typename TY>
 __global__ void __launch_bounds__(256)
 heads_gemm_kernel(const TX* __restrict__ x, long ldx, long hsx, const TW* __restrict__ w, TY* __restrict__ y, long ldy,
-                  long hsy, const float* __restrict__ gate, long ldg, int m, int n, int k, float alpha) {
+                  long hsy, ProductGate gate, QueryTurn turn, int m, int n, int k, float alpha) {
   __shared__ float xs[kHStep][kHTile + 4];
   __shared__ float ws[kHStep][kHTile + 4];
   const int tid = threadIdx.x;
   const int tx = tid % 16, ty = tid / 16;
   const int row0 = blockIdx.y * kHTile, col0 = blockIdx.x * kHTile;
   const int h = blockIdx.z;
+  if (col0 >= n) {   // the column of blocks behind the product's
+    turn_queries<TY>(turn, h, row0, m - row0 < kHTile ? m - row0 : kHTile);
+    return;
+  }
   const TX* xh = x + (size_t)h * hsx;
   const TW* wh = w + (size_t)h * n * k;
   float acc[4][4] = {};
@@ -148,12 +193,12 @@ heads_gemm_kernel(const TX* __restrict__ x, long ldx, long hsx, const TW* __rest
   for (int i = 0; i < 4; ++i) {
     const int r = row0 + ty * 4 + i;
     if (r >= m) continue;
-    float f = alpha;
-    if (gate) f *= 1.f / (1.f + expf(-gate[(size_t)r * ldg + h]));
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int c = col0 + tx * 4 + j;
-      if (c < n) y[(size_t)r * ldy + (size_t)h * hsy + c] = from_f32<TY>(acc[i][j] * f);
+      if (c < n)
+        y[(size_t)r * ldy + (size_t)h * hsy + c] =
+            from_f32<TY>(acc[i][j] * alpha * (gate.g ? gate_value(gate, r, h, c) : 1.f));
     }
   }
 }
@@ -167,10 +212,14 @@ constexpr int kHFewRows = 8;
 template <typename TX, typename TW, typename TY>
 __global__ void __launch_bounds__(256)
 heads_rows_kernel(const TX* __restrict__ x, long ldx, long hsx, const TW* __restrict__ w, TY* __restrict__ y, long ldy,
-                  long hsy, const float* __restrict__ gate, long ldg, int m, int n, int k, float alpha) {
+                  long hsy, ProductGate gate, QueryTurn turn, int m, int n, int k, float alpha) {
   const int lane = threadIdx.x % kWave;
   const int col = blockIdx.x * (256 / kWave) + threadIdx.x / kWave;
   const int h = blockIdx.y;
+  if (blockIdx.x * (256 / kWave) >= n) {   // the block behind the product's
+    turn_queries<TY>(turn, h, 0, m);
+    return;
+  }
   if (col >= n) return;
   const TX* xh = x + (size_t)h * hsx;
   const TW* wr = w + ((size_t)h * n + col) * k;
@@ -187,33 +236,52 @@ heads_rows_kernel(const TX* __restrict__ x, long ldx, long hsx, const TW* __rest
   for (int r = 0; r < kHFewRows; ++r) {
     if (r >= m) continue;
     const float total = wave_sum(acc[r]);
-    if (lane == 0) {
-      float f = alpha;
-      if (gate) f *= 1.f / (1.f + expf(-gate[(size_t)r * ldg + h]));
-      y[(size_t)r * ldy + (size_t)h * hsy + col] = from_f32<TY>(total * f);
-    }
+    if (lane == 0)
+      y[(size_t)r * ldy + (size_t)h * hsy + col] =
+          from_f32<TY>(total * alpha * (gate.g ? gate_value(gate, r, h, col) : 1.f));
   }
 }
 
+// The options of a per-head product from the host's plain arguments; false where they do not fit together.
+static bool product_options(const float* gate, long ldg, int hsg, int csg, const float* qx, long ldqx, long hsqx, void* qout,
+                            long ldqo, long hsqo, int rot, int rot_dims, const double* freq, float mult, float scale,
+                            const int* positions, ProductGate* g, QueryTurn* q) {
+  if (gate != nullptr && (ldg < 0 || hsg < 0 || csg < 0)) return false;
+  *g = ProductGate{gate, ldg, hsg, csg};
+  if (rot < 0 || rot_dims < 0 || rot_dims > rot || (rot_dims & 1)) return false;
+  if (rot > 0 && (qx == nullptr || qout == nullptr || positions == nullptr)) return false;
+  if (rot_dims > 0 && freq == nullptr) return false;
+  *q = QueryTurn{qx, qout, ldqx, hsqx, ldqo, hsqo, freq, positions, rot, rot_dims, mult, scale};
+  return true;
+}
+
 ATOM_EXPORT int atom_heads_gemm(const void* x, int x_dtype, long ldx, long hsx, const void* w, int w_dtype, void* y,
-                                int y_dtype, long ldy, long hsy, const float* gate, long ldg, int heads, int m, int n,
-                                int k, float alpha, hipStream_t stream) {
+                                int y_dtype, long ldy, long hsy, const float* gate, long ldg, int hsg, int csg,
+                                const float* qx, long ldqx, long hsqx, void* qout, long ldqo, long hsqo, int rot,
+                                int rot_dims, const double* freq, float mult, float scale, const int* positions, int heads,
+                                int m, int n, int k, float alpha, hipStream_t stream) {
   if (m < 0 || n <= 0 || k <= 0 || heads <= 0 || heads > 65535) return ATOM_BAD_SHAPE;
   if (x == nullptr || w == nullptr || y == nullptr) return ATOM_BAD_SHAPE;
   if ((unsigned)x_dtype > 1u || (unsigned)w_dtype > 1u || (unsigned)y_dtype > 1u) return ATOM_BAD_DTYPE;
+  ProductGate g;
+  QueryTurn q;
+  if (!product_options(gate, ldg, hsg, csg, qx, ldqx, hsqx, qout, ldqo, hsqo, rot, rot_dims, freq, mult, scale, positions,
+                       &g, &q))
+    return ATOM_BAD_SHAPE;
   if (m == 0) return ATOM_OK;
   const bool few = m <= kHFewRows;
-  dim3 grid((n + kHTile - 1) / kHTile, (m + kHTile - 1) / kHTile, heads), block(256);
-  if (few) grid = dim3((n + 3) / 4, heads, 1);
+  const int extra = rot > 0 ? 1 : 0;
+  dim3 grid((n + kHTile - 1) / kHTile + extra, (m + kHTile - 1) / kHTile, heads), block(256);
+  if (few) grid = dim3((n + 3) / 4 + extra, heads, 1);
   if (grid.y > 65535) return ATOM_TOO_LARGE;
 #define LAUNCH(TX, TW, TY)                                                                                          \
   do {                                                                                                              \
     if (few)                                                                                                        \
       hipLaunchKernelGGL((heads_rows_kernel<TX, TW, TY>), grid, block, 0, stream, (const TX*)x, ldx, hsx, (const TW*)w, \
-                         (TY*)y, ldy, hsy, gate, ldg, m, n, k, alpha);                                              \
+                         (TY*)y, ldy, hsy, g, q, m, n, k, alpha);                                                   \
     else                                                                                                            \
       hipLaunchKernelGGL((heads_gemm_kernel<TX, TW, TY>), grid, block, 0, stream, (const TX*)x, ldx, hsx, (const TW*)w, \
-                         (TY*)y, ldy, hsy, gate, ldg, m, n, k, alpha);                                              \
+                         (TY*)y, ldy, hsy, g, q, m, n, k, alpha);                                                   \
   } while (0)
   switch (x_dtype * 4 + w_dtype * 2 + y_dtype) {
     case 0: LAUNCH(float, float, float); break;
@@ -395,9 +463,13 @@ __device__ __forceinline__ void hg_load8_split(const float* p, bool ok, hg_bf16x
 template <typename TX, typename TY, bool SPLIT = false>
 __global__ void __launch_bounds__(256)
 heads_gemm_mfma_kernel(const TX* __restrict__ x, long ldx, long hsx, const bf16_t* __restrict__ w, TY* __restrict__ y,
-                       long ldy, long hsy, const float* __restrict__ gate, long ldg, int m, int n, int k, float alpha) {
+                       long ldy, long hsy, ProductGate gate, QueryTurn turn, int m, int n, int k, float alpha) {
   const int tid = threadIdx.x, wave = tid / kWave, lane = tid % kWave, r = lane % 16, g = lane / 16;
   const int h = blockIdx.z;
+  if (blockIdx.x * 64 >= n) {   // the column of blocks behind the product's
+    turn_queries<TY>(turn, h, blockIdx.y * 64, m - (int)blockIdx.y * 64 < 64 ? m - (int)blockIdx.y * 64 : 64);
+    return;
+  }
   const int row0 = blockIdx.y * 64 + (wave / 2) * 32;
   const int col0 = blockIdx.x * 64 + (wave % 2) * 32;
   const TX* xrow[2];
@@ -448,14 +520,14 @@ heads_gemm_mfma_kernel(const TX* __restrict__ x, long ldx, long hsx, const bf16_
   for (int rt = 0; rt < 2; ++rt) {
     const int row = row0 + rt * 16 + r;
     if (row >= m) continue;
-    float f = alpha;
-    if (gate) f *= 1.f / (1.f + expf(-gate[(size_t)row * ldg + h]));
 #pragma unroll
     for (int ct = 0; ct < 2; ++ct) {
       const int col = col0 + ct * 16 + 4 * g;
 #pragma unroll
       for (int i = 0; i < 4; ++i)
-        if (col + i < n) y[(size_t)row * ldy + (size_t)h * hsy + col + i] = from_f32<TY>(acc[ct][rt][i] * f);
+        if (col + i < n)
+          y[(size_t)row * ldy + (size_t)h * hsy + col + i] =
+              from_f32<TY>(acc[ct][rt][i] * alpha * (gate.g ? gate_value(gate, row, h, col + i) : 1.f));
     }
   }
 }
@@ -467,32 +539,35 @@ ATOM_EXPORT int atom_heads_gemm_mfma_supports(int x_dtype, int w_dtype, long x_o
 }
 
 ATOM_EXPORT int atom_heads_gemm_mfma(const void* x, int x_dtype, long ldx, long hsx, const void* w, void* y, int y_dtype,
-                                     long ldy, long hsy, const float* gate, long ldg, int heads, int m, int n, int k,
-                                     float alpha, int split, hipStream_t stream) {
+                                     long ldy, long hsy, const float* gate, long ldg, int hsg, int csg, const float* qx,
+                                     long ldqx, long hsqx, void* qout, long ldqo, long hsqo, int rot, int rot_dims,
+                                     const double* freq, float mult, float scale, const int* positions, int heads, int m,
+                                     int n, int k, float alpha, int split, hipStream_t stream) {
   if (m < 0 || n <= 0 || k <= 0 || heads <= 0 || heads > 65535 || (k % 8)) return ATOM_BAD_SHAPE;
   if (split && x_dtype != ATOM_F32) return ATOM_UNSUPPORTED;   // only a float32 input has pieces to split into
   if (x == nullptr || w == nullptr || y == nullptr) return ATOM_BAD_SHAPE;
   if ((unsigned)x_dtype > 1u || (unsigned)y_dtype > 1u) return ATOM_BAD_DTYPE;
+  ProductGate g;
+  QueryTurn q;
+  if (!product_options(gate, ldg, hsg, csg, qx, ldqx, hsqx, qout, ldqo, hsqo, rot, rot_dims, freq, mult, scale, positions,
+                       &g, &q))
+    return ATOM_BAD_SHAPE;
   if (m == 0) return ATOM_OK;
-  dim3 grid((n + 63) / 64, (m + 63) / 64, heads), block(256);
+  dim3 grid((n + 63) / 64 + (rot > 0 ? 1 : 0), (m + 63) / 64, heads), block(256);
   if (grid.y > 65535) return ATOM_TOO_LARGE;
-#define LAUNCH(TX, TY)                                                                                            \
-  hipLaunchKernelGGL((heads_gemm_mfma_kernel<TX, TY>), grid, block, 0, stream, (const TX*)x, ldx, hsx,           \
-                     (const bf16_t*)w, (TY*)y, ldy, hsy, gate, ldg, m, n, k, alpha)
+#define LAUNCH(TX, TY, SPLIT)                                                                                       \
+  hipLaunchKernelGGL((heads_gemm_mfma_kernel<TX, TY, SPLIT>), grid, block, 0, stream, (const TX*)x, ldx, hsx,      \
+                     (const bf16_t*)w, (TY*)y, ldy, hsy, g, q, m, n, k, alpha)
   if (split) {
-    if (y_dtype == ATOM_F32)
-      hipLaunchKernelGGL((heads_gemm_mfma_kernel<float, float, true>), grid, block, 0, stream, (const float*)x, ldx, hsx,
-                         (const bf16_t*)w, (float*)y, ldy, hsy, gate, ldg, m, n, k, alpha);
-    else
-      hipLaunchKernelGGL((heads_gemm_mfma_kernel<float, bf16_t, true>), grid, block, 0, stream, (const float*)x, ldx, hsx,
-                         (const bf16_t*)w, (bf16_t*)y, ldy, hsy, gate, ldg, m, n, k, alpha);
+    if (y_dtype == ATOM_F32) LAUNCH(float, float, true);
+    else LAUNCH(float, bf16_t, true);
     return launch_status();
   }
   switch (x_dtype * 2 + y_dtype) {
-    case 0: LAUNCH(float, float); break;
-    case 1: LAUNCH(float, bf16_t); break;
-    case 2: LAUNCH(bf16_t, float); break;
-    default: LAUNCH(bf16_t, bf16_t); break;
+    case 0: LAUNCH(float, float, false); break;
+    case 1: LAUNCH(float, bf16_t, false); break;
+    case 2: LAUNCH(bf16_t, float, false); break;
+    default: LAUNCH(bf16_t, bf16_t, false); break;
   }
 #undef LAUNCH
   return launch_status();

@@ -96,6 +96,23 @@ class AttentionMeta:
     tiles_by_rows: dict | None = None
 
 
+@dataclass
+class QueryTurn:
+    """The rotated parts of queries, which a per-head product (``HipKernels.heads_gemm``) turns and writes beside its
+    output: head h's ``rot`` entries of token t at ``x_offset + t * ldx + h * hsx`` of its float32 input, the first
+    ``rot_dims`` of them rotated in neighbouring pairs by ``positions[t] * freq``, times ``scale``, go to ``y_offset + t
+    * ldy + h * hsy`` of its output."""
+
+    x_offset: int
+    y_offset: int
+    rot: int
+    rot_dims: int
+    freq: torch.Tensor | None
+    mult: float
+    scale: float
+    positions: torch.Tensor
+
+
 class DeferredSum:
     """A matrix product that is still a sum of slices: ``partial`` float32 [splits, rows, width], plus an
     optional bias over the width.  The skinny product leaves its result like this when it cuts K; the
@@ -1018,39 +1035,51 @@ class HipKernels:
 
     # ------------------------------------------------------------------ attention over a cache of latents
 
-    def latent_prepare(self, proj, q_off: int, kv_off: int, heads: int, dim: int, rot: int, rank: int, rot_dims: int,
-                       norm_weight, eps: float, freq, mult: float, positions, slots, pages, q_abs, q_scale: float):
-        """From the float32 product ``proj`` [tokens, *] (queries of ``heads`` x (dim + rot) at ``q_off``, the
-        down-projection of rank + rot at ``kv_off``): the RMS-normed latent and the rotated shared key part go to
-        row ``slots[t]`` of ``pages`` (None: no write), the queries' rotated parts, times ``q_scale``, to
-        ``q_abs[t, h, rank:]``."""
+    def latent_prepare(self, proj, pages, slots, positions, kv_off: int, rank: int, rot: int, norm_weight, eps: float,
+                       freq=None, rot_dims: int = 0, mult: float = 1.0, query=None):
+        """From the float32 product ``proj`` [tokens, *]: the RMS-normed latent (``rank`` entries at ``kv_off``) and the
+        rotated shared key part (the ``rot`` entries after it) go to row ``slots[t]`` of ``pages`` (``slots`` None: no
+        keys are projected here).  ``query`` = (offset, weight, out): the latent that queries are projected up from,
+        RMS-normed with ``weight`` into ``out`` [tokens, its size].  ``eps`` is both norms'."""
         tokens, ld = proj.shape
-        width = rank + rot
         self._check("projections", proj, torch.float32)
-        self._check("latent norm weight", norm_weight, torch.float32, (rank,))
-        self._check("positions", positions, torch.int32, (tokens,))
-        self._check("absorbed queries", q_abs, (torch.float32, torch.bfloat16), (tokens, heads, width))
-        if rot_dims:
-            self._check("rotation frequencies", freq, torch.float64, (rot_dims // 2,))
+        cq_off, cq_rank, cq_weight, cq = 0, 0, None, None
+        if query is not None:
+            cq_off, cq_weight, cq = query
+            cq_rank = cq.shape[1]
+            self._check("query latent norm weight", cq_weight, torch.float32, (cq_rank,))
+            self._check("query latent", cq, (torch.float32, torch.bfloat16), (tokens, cq_rank))
+            if cq_off < 0 or cq_off + cq_rank > ld:
+                raise KernelError("latent_prepare: the query latent's columns are not in the product")
         if slots is not None:
+            self._check("latent norm weight", norm_weight, torch.float32, (rank,))
+            self._check("positions", positions, torch.int32, (tokens,))
             self._check("slot mapping", slots, torch.int32, (tokens,))
-            self._check("latent pages", pages, q_abs.dtype, (None, None, width))
+            self._check("latent pages", pages, cq.dtype if cq is not None else (torch.float32, torch.bfloat16),
+                        (None, None, rank + rot))
+            if kv_off < 0 or kv_off + rank + rot > ld:
+                raise KernelError("latent_prepare: the keys' columns are not in the product")
+            if rot_dims:
+                self._check("rotation frequencies", freq, torch.float64, (rot_dims // 2,))
+        elif query is None:
+            return
         self._done("latent_prepare", self.lib.atom_latent_prepare(
-            _ptr(proj), ld, q_off, kv_off, heads, dim, rot, rank, rot_dims, _ptr(norm_weight), ctypes.c_float(eps),
-            _ptr(freq) if rot_dims else None, ctypes.c_float(mult), _ptr(positions), _ptr(slots),
-            _ptr(pages) if slots is not None else None, _ptr(q_abs), self._code(q_abs), tokens, ctypes.c_float(q_scale),
-            self._stream()))
-        return q_abs
+            _ptr(proj), ld, cq_off, cq_rank, _ptr(cq_weight), _ptr(cq), kv_off, rank, rot, rot_dims,
+            _ptr(norm_weight) if slots is not None else None, ctypes.c_float(eps), _ptr(freq) if rot_dims else None,
+            ctypes.c_float(mult), _ptr(positions), _ptr(slots), _ptr(pages) if slots is not None else None,
+            self._code(cq if cq is not None else pages), tokens, self._stream()))
 
     def heads_gemm(self, x, x_offset: int, ldx: int, hsx: int, weight, y, y_offset: int, ldy: int, hsy: int, heads: int,
                    m: int, n: int, k: int, alpha: float = 1.0, gate=None, gate_offset: int = 0, ldg: int = 0,
-                   exact: bool = False):
+                   gate_entries: bool = False, exact: bool = False, turn: QueryTurn | None = None):
         """One small product per head: ``y[t, h, :n] = alpha * x[t, h, :k] @ weight[h].T`` (times
-        ``sigmoid(gate[t, h])`` when given), with ``x`` and ``y`` addressed as flat arrays: element (t, h, i) of x
-        sits at ``x_offset + t * ldx + h * hsx + i``.  ``weight`` is [heads, n, k].  ``exact``: a float32 input is
+        ``sigmoid(gate[t, h])`` when given, or with ``gate_entries`` ``sigmoid(gate[t, h * n + c])`` for column c),
+        with ``x`` and ``y`` addressed as flat arrays: element (t, h, i) of x sits at
+        ``x_offset + t * ldx + h * hsx + i``.  ``weight`` is [heads, n, k].  ``exact``: a float32 input is
         multiplied as it is, not rounded for the matrix cores: float32 multiply-adds for few rows or float32
         weights, and for many rows with bfloat16 weights the matrix cores on the input's three bfloat16 pieces,
-        whose products with a bfloat16 weight are exact."""
+        whose products with a bfloat16 weight are exact.  ``turn``: rotated parts of queries that the launch turns and
+        writes beside its product (see ``QueryTurn``; ``x`` and ``y`` are the tensors it names offsets in)."""
         self._check("per-head input", x, (torch.float32, torch.bfloat16))
         self._check("per-head weight", weight, (torch.float32, torch.bfloat16), (heads, n, k))
         self._check("per-head out", y, (torch.float32, torch.bfloat16))
@@ -1062,9 +1091,26 @@ class HipKernels:
         gp = None
         if gate is not None:
             self._check("per-head gate", gate, torch.float32)
-            if m and gate_offset + (m - 1) * ldg + heads > gate.numel():
+            if m and gate_offset + (m - 1) * ldg + heads * (n if gate_entries else 1) > gate.numel():
                 raise KernelError("heads_gemm: the gate is smaller than its strides say")
             gp = ctypes.c_void_p(gate.data_ptr() + 4 * gate_offset)
+        options = [gp, ctypes.c_long(ldg), n if gate_entries else 1, 1 if gate_entries else 0]
+        if turn is not None and turn.rot:
+            self._check("queries to turn", x, torch.float32)
+            self._check("positions", turn.positions, torch.int32, (m,))
+            if turn.rot_dims:
+                self._check("rotation frequencies", turn.freq, torch.float64, (turn.rot_dims // 2,))
+            if m and (turn.x_offset + (m - 1) * ldx + (heads - 1) * hsx + turn.rot > x.numel()
+                      or turn.y_offset + (m - 1) * ldy + (heads - 1) * hsy + turn.rot > y.numel()):
+                raise KernelError("heads_gemm: the queries to turn do not lie in the product's tensors")
+            options += [ctypes.c_void_p(x.data_ptr() + x.element_size() * turn.x_offset), ctypes.c_long(ldx),
+                        ctypes.c_long(hsx), ctypes.c_void_p(y.data_ptr() + y.element_size() * turn.y_offset),
+                        ctypes.c_long(ldy), ctypes.c_long(hsy), turn.rot, turn.rot_dims,
+                        _ptr(turn.freq) if turn.rot_dims else None, ctypes.c_float(turn.mult), ctypes.c_float(turn.scale),
+                        _ptr(turn.positions)]
+        else:
+            zero = ctypes.c_long(0)
+            options += [None, zero, zero, None, zero, zero, 0, 0, None, ctypes.c_float(1.0), ctypes.c_float(1.0), None]
         xp = ctypes.c_void_p(x.data_ptr() + x.element_size() * x_offset)
         yp = ctypes.c_void_p(y.data_ptr() + y.element_size() * y_offset)
         split = bool(exact and x.dtype == torch.float32)
@@ -1074,13 +1120,13 @@ class HipKernels:
             # many rows: the same product on the matrix cores (a float32 input is rounded to bfloat16 on the way in)
             self._done("heads_gemm_mfma", self.lib.atom_heads_gemm_mfma(
                 xp, self._code(x), ctypes.c_long(ldx), ctypes.c_long(hsx), _ptr(weight), yp, self._code(y),
-                ctypes.c_long(ldy), ctypes.c_long(hsy), gp, ctypes.c_long(ldg), heads, m, n, k, ctypes.c_float(alpha),
-                int(split), self._stream()))
+                ctypes.c_long(ldy), ctypes.c_long(hsy), *options, heads, m, n, k, ctypes.c_float(alpha), int(split),
+                self._stream()))
             return y
         self._done("heads_gemm", self.lib.atom_heads_gemm(
             xp, self._code(x), ctypes.c_long(ldx), ctypes.c_long(hsx), _ptr(weight), self._code(weight), yp,
-            self._code(y), ctypes.c_long(ldy), ctypes.c_long(hsy), gp, ctypes.c_long(ldg), heads, m, n, k,
-            ctypes.c_float(alpha), self._stream()))
+            self._code(y), ctypes.c_long(ldy), ctypes.c_long(hsy), *options, heads, m, n, k, ctypes.c_float(alpha),
+            self._stream()))
         return y
 
     def latent_parts(self, meta: AttentionMeta, heads: int, window: int | None) -> int:
@@ -1780,23 +1826,31 @@ class HipKernels:
             ctypes.c_long(stride), self._stream()))
         return out
 
-    def router_choose(self, logits, correction, top: int, renormalize: bool = False):
-        """(ids int32 [tokens, top], weights float32 [tokens, top]) from float32 router logits: scores are
-        sigmoids; the choice adds ``correction`` to them, the weights do not."""
+    def router_choose(self, logits, correction, top: int, renormalize: bool = False, score: str = "sigmoid",
+                      eps: float = 0.0, scale: float = 1.0):
+        """(ids int32 [tokens, top], weights float32 [tokens, top]) from float32 router logits: scores are their
+        sigmoids or (``score`` "softmax") their softmax over all of a token's logits; the choice adds ``correction`` to
+        them, the weights do not.  A weight is its score, divided with ``renormalize`` by the chosen scores' sum + eps,
+        times ``scale``."""
         tokens, experts = logits.shape
         self._check("router logits", logits, torch.float32)
         if correction is not None:
             self._check("router correction", correction, torch.float32, (experts,))
+        if score not in ("sigmoid", "softmax"):
+            raise KernelError(f"router: unknown score {score!r}")
         ids = torch.empty((tokens, top), dtype=torch.int32, device=logits.device)
         weights = torch.empty((tokens, top), dtype=torch.float32, device=logits.device)
         self._done("router_choose", self.lib.atom_router_choose(
-            _ptr(logits), _ptr(correction), _ptr(ids), _ptr(weights), tokens, experts, top, int(bool(renormalize)),
-            self._stream()))
+            _ptr(logits), _ptr(correction), _ptr(ids), _ptr(weights), tokens, experts, top, int(score == "softmax"),
+            int(bool(renormalize)), ctypes.c_float(eps), ctypes.c_float(scale), self._stream()))
         return ids, weights
 
-    def experts_forward(self, x, gate_up, down, ids, weights, activation: str = "silu"):
-        """``sum_k weights[t, k] * down[e] (act(gate[e] x) * (up[e] x))`` with e = ids[t, k].  ``gate_up``
-        [experts, 2 ff, width] (gate rows, then up rows), ``down`` [experts, width, ff]."""
+    def experts_forward(self, x, gate_up, down, ids, weights, activation: str = "silu", limit: float | None = None,
+                        slope: float = 1.0, shift: float = 0.0):
+        """``sum_k weights[t, k] * down[e] f(gate[e] x, up[e] x)`` with e = ids[t, k] and ``f(g, u) = act(g) * u``.
+        ``gate_up`` [experts, 2 ff, width] (gate rows, then up rows), ``down`` [experts, width, ff].  An id from
+        ``experts`` on is an identity expert, whose result is x itself.  SiLU takes three constants:
+        ``f(g, u) = g' * sigmoid(slope * g') * (u' + shift)``, g' being at most ``limit`` and u' within it."""
         x = self.materialize(x)
         tokens, width = x.shape
         experts, two_ff, _ = gate_up.shape
@@ -1809,6 +1863,10 @@ class HipKernels:
         self._check("expert weights", weights, torch.float32, (tokens, top))
         if activation not in self._ACTIVATIONS:
             raise KernelError(f"experts: unknown activation {activation!r}")
+        if activation != "silu" and (limit is not None or slope != 1.0 or shift != 0.0):
+            raise KernelError("experts: limit, slope and shift are SiLU's")
+        gate = [self._ACTIVATIONS[activation], ctypes.c_float(math.inf if limit is None else limit),
+                ctypes.c_float(slope), ctypes.c_float(shift)]
         if (x.dtype == torch.bfloat16 and gate_up.dtype == torch.bfloat16 and tokens * top >= self.grouped_experts_from
                 and self.lib.atom_experts_grouped_supports(ff, width, experts)):
             tiles = self.lib.atom_experts_grouped_tiles(tokens * top, experts)
@@ -1819,16 +1877,16 @@ class HipKernels:
             self._done("experts_grouped", self.lib.atom_experts_grouped(
                 _ptr(x), _ptr(gate_up), _ptr(down), _ptr(ids), _ptr(weights), _ptr(ints),
                 ctypes.c_void_p(ints.data_ptr() + 4 * tiles), ctypes.c_void_p(ints.data_ptr() + 4 * tiles * 65), _ptr(act),
-                _ptr(rows), _ptr(y), tokens, top, experts, ff, width, self._ACTIVATIONS[activation], self._stream()))
+                _ptr(rows), _ptr(y), tokens, top, experts, ff, width, *gate, self._stream()))
             return y
         act = torch.empty((tokens * top, ff), dtype=x.dtype, device=x.device)
         self._done("experts_gate_up", self.lib.atom_experts_gate_up(
-            _ptr(x), _ptr(gate_up), self._code(gate_up), _ptr(ids), _ptr(act), self._code(x), tokens, top, ff, width,
-            self._ACTIVATIONS[activation], self._stream()))
+            _ptr(x), _ptr(gate_up), self._code(gate_up), _ptr(ids), _ptr(act), self._code(x), tokens, top, experts, ff,
+            width, *gate, self._stream()))
         y = torch.empty((tokens, width), dtype=x.dtype, device=x.device)
         self._done("experts_down", self.lib.atom_experts_down(
-            _ptr(act), _ptr(down), self._code(down), _ptr(ids), _ptr(weights), _ptr(y), self._code(x), tokens, top, ff,
-            width, self._stream()))
+            _ptr(x), _ptr(act), _ptr(down), self._code(down), _ptr(ids), _ptr(weights), _ptr(y), self._code(x), tokens, top,
+            experts, ff, width, self._stream()))
         return y
 
     def sample(self, logits, temperatures, out, top_ks=None, top_ps=None, noise=None, seeds=None, counters=None,

@@ -30,7 +30,7 @@ def _mixer(cfg: LotoraxConfig, layer: dict) -> PartChoice:
         return PartChoice("latent_attention", {
             "hidden_size": cfg.hidden_size, "num_heads": m["heads"], "head_dim": m["dim"], "rot_dim": m["rot_dim"],
             "value_dim": m["vdim"], "kv_rank": m["kv_rank"], "scale": m["scale"], "norm_eps": cfg.norm_eps,
-            "position_encoding": rope, "sink": True, "gate": True})
+            "position_encoding": rope, "sink": True, "gate": "head"})
     return PartChoice("gated_delta", {
         "hidden_size": cfg.hidden_size, "num_heads": m["heads"], "num_kv_heads": m["kv_heads"], "head_dim": m["dim"],
         "value_dim": m["vdim"], "conv_taps": m["conv"], "norm_eps": cfg.norm_eps})

@@ -10,6 +10,7 @@ from dataclasses import dataclass, field
 
 import torch
 
+from ..cache.kinds import kind_of
 from ..parts.base import BLOCKS, EMBEDDINGS, HEADS, JOINS, NORMS, Part, PartChoice
 
 
@@ -83,10 +84,7 @@ class CausalLM(Part):
                     raise ValueError(f"run {i} reads the cache of run {run.reads_run}, which does not come before it")
                 if self.order[run.reads_run].reads_run is not None:
                     raise ValueError(f"run {i} reads run {run.reads_run}, which has no cache of its own")
-                a = self.blocks[run.layer].mixer.cache_need()
-                b = self.blocks[self.order[run.reads_run].layer].mixer.cache_need()
-                if a != b:
-                    raise ValueError(f"run {i} cannot read the cache of run {run.reads_run}: {a} differs from {b}")
+        self.memory_needs()      # raises where a run cannot read the memory its order names
         self.ignorable = set(spec.ignorable)
         if spec.tie_word_embeddings:
             self.ignorable.add(f"{spec.head_prefix}.weight")
@@ -98,6 +96,22 @@ class CausalLM(Part):
     def children(self):
         return [self.embedding, *self.tables.values(), *([self.join] if self.join is not None else []), *self.blocks,
                 self.final_norm, self.head]
+
+    def memory_needs(self) -> list:
+        """What every run of the order keeps between steps (None: nothing).  A run's memory is kept for all who read it:
+        the need of a run that others read is joined with theirs, and a reading run is listed with its owner's."""
+        needs = [self.blocks[run.layer].mixer.cache_need() for run in self.order]
+        for i, run in enumerate(self.order):
+            if run.reads_run is None:
+                continue
+            owner = needs[run.reads_run]
+            try:
+                if type(owner) is not type(needs[i]):
+                    raise ValueError(f"{needs[i]} differs from {owner}")
+                needs[run.reads_run] = kind_of(owner).joined(owner, needs[i]) if owner is not None else None
+            except ValueError as e:
+                raise ValueError(f"run {i} cannot read the cache of run {run.reads_run}: {e}") from None
+        return [needs[i if run.reads_run is None else run.reads_run] for i, run in enumerate(self.order)]
 
     def drops(self, name: str) -> str | None:
         """Why a checkpoint tensor that no parameter names is left aside without an error, or None if it

@@ -1,10 +1,15 @@
 """A feed-forward of routed experts: every token runs ``top`` of ``experts`` small gated feed-forwards and takes
 the weighted sum of their outputs.
 
-The router's logits are a float32 product; the scores are their sigmoids.  A per-expert ``correction`` is added to
-the scores for the choice only (a load-balancing bias that leaves the weights alone); the weights are the chosen
-experts' scores, renormalised to sum to one only when asked.  Experts have no biases; their matrices are stacked
-[experts, 2 ff, width] (gate rows, then up rows) and [experts, width, ff].
+The router's logits are a float32 product; the scores are their sigmoids, or their softmax over all of a token's logits.
+A per-expert ``correction`` is added to the scores for the choice only (a load-balancing bias that leaves the weights
+alone); the weights are the chosen experts' scores, with ``renormalize`` divided by their sum + ``weight_eps``, times
+``weight_scale``.  The router's last ``identity`` outputs stand for experts without matrices, whose output is the input
+itself.
+
+Experts have no biases; their matrices are stacked [experts, 2 ff, width] (gate rows, then up rows) and [experts, width,
+ff].  An expert is ``W_down (act(W_gate x) * (W_up x))``; SiLU experts may name ``limit``, ``slope`` and ``shift``:
+``W_down (g sigmoid(slope g) (u + shift))`` with ``g = min(W_gate x, limit)`` and ``u = W_up x`` within ``limit``.
 """
 
 from __future__ import annotations
@@ -13,15 +18,24 @@ from .base import FEED_FORWARDS, FeedForward, ParamSpec
 
 
 class RoutedExperts(FeedForward):
+    SCORES = ("sigmoid", "softmax")
+
     def __init__(self, hidden_size: int, expert_size: int, num_experts: int, top: int, activation: str = "silu",
-                 correction: bool = True, renormalize: bool = False, prefix: str = "",
-                 names: dict[str, str] | None = None):
+                 correction: bool = True, renormalize: bool = False, score: str = "sigmoid", weight_eps: float = 0.0,
+                 weight_scale: float = 1.0, identity: int = 0, limit: float | None = None, slope: float = 1.0,
+                 shift: float = 0.0, prefix: str = "", names: dict[str, str] | None = None):
         super().__init__(prefix)
-        if not 0 < top <= num_experts:
-            raise ValueError(f"a token cannot use {top} of {num_experts} experts")
+        if not 0 < top <= num_experts + identity or identity < 0 or num_experts <= 0:
+            raise ValueError(f"a token cannot use {top} of {num_experts} + {identity} experts")
+        if score not in self.SCORES:
+            raise ValueError(f"router scores are one of {self.SCORES}, got {score!r}")
         self.hidden_size, self.expert_size, self.num_experts, self.top = hidden_size, expert_size, num_experts, top
+        self.identity = int(identity)
         self.activation = activation
-        self.has_correction, self.renormalize = bool(correction), bool(renormalize)
+        self.gate_options = {"limit": limit, "slope": float(slope), "shift": float(shift)}
+        self.has_correction = bool(correction)
+        self.weight_rule = {"renormalize": bool(renormalize), "score": score, "eps": float(weight_eps),
+                            "scale": float(weight_scale)}
         self.names = {"router": "router", "correction": "correction", "expert": "e{}", "gate": "gate", "up": "up",
                       "down": "down", **(names or {})}
         self.gate_up = self.down = None
@@ -34,12 +48,13 @@ class RoutedExperts(FeedForward):
             gate_up += [(f"{ex}.{n['gate']}", f), (f"{ex}.{n['up']}", f)]
             down.append((f"{ex}.{n['down']}", h))
         specs = {
-            "router.weight": ParamSpec.single(n["router"], (self.num_experts, h)),
+            "router.weight": ParamSpec.single(n["router"], (self.num_experts + self.identity, h)),
             "gate_up.weight": ParamSpec.stacked(gate_up, (h,)),
             "down.weight": ParamSpec.stacked(down, (f,)),
         }
         if self.has_correction:
-            specs["correction"] = ParamSpec.single(n["correction"], (self.num_experts,), kind="vector")
+            specs["correction"] = ParamSpec.single(n["correction"], (self.num_experts + self.identity,),
+                                                      kind="vector")
         return specs
 
     def finalize(self, device, dtype):
@@ -49,8 +64,8 @@ class RoutedExperts(FeedForward):
     def forward(self, ctx, x):
         ops = ctx.ops
         logits = ops.linear_f32(x, self.params["router.weight"])
-        ids, weights = ops.router_choose(logits, self.p("correction"), self.top, self.renormalize)
-        return ops.experts_forward(x, self.gate_up, self.down, ids, weights, self.activation)
+        ids, weights = ops.router_choose(logits, self.p("correction"), self.top, **self.weight_rule)
+        return ops.experts_forward(x, self.gate_up, self.down, ids, weights, self.activation, **self.gate_options)
 
 
 FEED_FORWARDS.register("routed_experts", RoutedExperts)

@@ -267,45 +267,51 @@ class PlainKernels:
     def linear_f32(self, x, weight, bias=None):
         return self.linear(x, weight, bias, out_dtype=torch.float32)
 
-    def latent_prepare(self, proj, q_off, kv_off, heads, dim, rot, rank, rot_dims, norm_weight, eps, freq, mult,
-                       positions, slots, pages, q_abs, q_scale):
-        T = proj.shape[0]
+    @staticmethod
+    def _turn(x, positions, freq, rot_dims, mult):
+        """x [T, ..., n]: neighbouring pairs of the first ``rot_dims`` entries turned by position * freq."""
+        if not rot_dims:
+            return x
+        ang = positions.to(WIDE)[:, None] * freq.to(WIDE)[None, :]
+        c, s_ = torch.cos(ang) * mult, torch.sin(ang) * mult
+        while c.dim() < x.dim():
+            c, s_ = c.unsqueeze(1), s_.unsqueeze(1)
+        out = x.clone()
+        u, v = x[..., 0:rot_dims:2], x[..., 1:rot_dims:2]
+        out[..., 0:rot_dims:2] = u * c - v * s_
+        out[..., 1:rot_dims:2] = v * c + u * s_
+        return out
+
+    def latent_prepare(self, proj, pages, slots, positions, kv_off, rank, rot, norm_weight, eps, freq=None, rot_dims=0,
+                       mult=1.0, query=None):
         p = proj.to(WIDE)
-        ang = positions.to(WIDE)[:, None] * freq.to(WIDE)[None, :] if rot_dims else None
-
-        def turn(x):   # x [T, ..., rot]
-            if not rot_dims:
-                return x
-            c, s_ = torch.cos(ang) * mult, torch.sin(ang) * mult
-            while c.dim() < x.dim():
-                c, s_ = c.unsqueeze(1), s_.unsqueeze(1)
-            out = x.clone()
-            u, v = x[..., 0:rot_dims:2], x[..., 1:rot_dims:2]
-            out[..., 0:rot_dims:2] = u * c - v * s_
-            out[..., 1:rot_dims:2] = v * c + u * s_
-            return out
-
-        q = p[:, q_off:q_off + heads * (dim + rot)].reshape(T, heads, dim + rot)
-        q_abs[:, :, rank:] = (turn(q[..., dim:]) * q_scale).to(q_abs.dtype)
+        if query is not None:
+            off, weight, out = query
+            out.copy_((pl.rms_unit(p[:, off:off + out.shape[1]], eps) * weight.to(WIDE)).to(out.dtype))
         if slots is not None:
             c = pl.rms_unit(p[:, kv_off:kv_off + rank], eps) * norm_weight.to(WIDE)
-            k = turn(p[:, kv_off + rank:kv_off + rank + rot])
+            k = self._turn(p[:, kv_off + rank:kv_off + rank + rot], positions, freq, rot_dims, mult)
             flat = pages.view(-1, rank + rot)
-            for t in range(T):
+            for t in range(proj.shape[0]):
                 if int(slots[t]) >= 0:
                     flat[int(slots[t])] = torch.cat((c[t], k[t])).to(pages.dtype)
-        return q_abs
 
     def heads_gemm(self, x, x_offset, ldx, hsx, weight, y, y_offset, ldy, hsy, heads, m, n, k, alpha=1.0, gate=None,
-                   gate_offset=0, ldg=0, exact=False):
+                   gate_offset=0, ldg=0, gate_entries=False, exact=False, turn=None):
         xf, yf = x.reshape(-1), y.view(-1)
         for h in range(heads):
             xs = torch.as_strided(xf, (m, k), (ldx, 1), x_offset + h * hsx).to(WIDE)
             r = alpha * (xs @ weight[h].to(WIDE).T)
-            if gate is not None:
+            if gate is not None and gate_entries:
+                r = r * torch.sigmoid(torch.as_strided(gate.reshape(-1), (m, n), (ldg, 1), gate_offset + h * n).to(WIDE))
+            elif gate is not None:
                 gv = torch.as_strided(gate.reshape(-1), (m,), (ldg,), gate_offset + h).to(WIDE)
                 r = r * torch.sigmoid(gv)[:, None]
             torch.as_strided(yf, (m, n), (ldy, 1), y_offset + h * hsy).copy_(r.to(y.dtype))
+            if turn is not None and turn.rot:
+                part = torch.as_strided(xf, (m, turn.rot), (ldx, 1), turn.x_offset + h * hsx).to(WIDE)
+                part = self._turn(part, turn.positions, turn.freq, turn.rot_dims, turn.mult) * turn.scale
+                torch.as_strided(yf, (m, turn.rot), (ldy, 1), turn.y_offset + h * hsy).copy_(part.to(y.dtype))
         return y
 
     def latent_attention(self, q_abs, pages, out, meta, rank, sink=None, window=None):
@@ -639,25 +645,31 @@ class PlainKernels:
         out.copy_((x.to(WIDE) * torch.sigmoid(g)).to(out.dtype))
         return out
 
-    def router_choose(self, logits, correction, top, renormalize=False):
-        s = torch.sigmoid(logits.to(WIDE))
+    def router_choose(self, logits, correction, top, renormalize=False, score="sigmoid", eps=0.0, scale=1.0):
+        z = logits.to(WIDE)
+        s = torch.sigmoid(z) if score == "sigmoid" else torch.softmax(z, dim=-1)
         pick = s + correction.to(WIDE) if correction is not None else s
         ids = torch.topk(pick, top, dim=-1).indices
         w = torch.gather(s, 1, ids)
         if renormalize:
-            w = w / w.sum(dim=-1, keepdim=True)
-        return ids.to(torch.int32), w.to(torch.float32)
+            w = w / (w.sum(dim=-1, keepdim=True) + eps)
+        return ids.to(torch.int32), (w * scale).to(torch.float32)
 
-    def experts_forward(self, x, gate_up, down, ids, weights, activation="silu"):
-        f = {"silu": pl.silu, "relu": torch.relu, "gelu_tanh": pl.gelu_tanh}[activation]
+    def experts_forward(self, x, gate_up, down, ids, weights, activation="silu", limit=None, slope=1.0, shift=0.0):
+        f = {"silu": lambda z: z * torch.sigmoid(slope * z), "relu": torch.relu, "gelu_tanh": pl.gelu_tanh}[activation]
         xs = x.to(WIDE)
         y = torch.zeros(xs.shape, dtype=WIDE)
         ff = gate_up.shape[1] // 2
         for t in range(xs.shape[0]):
             for k in range(ids.shape[1]):
                 e = int(ids[t, k])
-                both = gate_up[e].to(WIDE) @ xs[t]
-                y[t] += float(weights[t, k]) * (down[e].to(WIDE) @ (f(both[:ff]) * both[ff:]))
+                if e >= gate_up.shape[0]:
+                    y[t] += float(weights[t, k]) * xs[t]
+                    continue
+                g, u = (gate_up[e].to(WIDE) @ xs[t]).split(ff)
+                if limit is not None:
+                    g, u = torch.clamp(g, max=limit), torch.clamp(u, -limit, limit)
+                y[t] += float(weights[t, k]) * (down[e].to(WIDE) @ (f(g) * (u + shift)))
         return y.to(x.dtype)
 
     def exponential_noise(self, seeds, counters, vocab):

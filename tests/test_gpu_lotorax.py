@@ -13,7 +13,7 @@ import plain_lotorax as pl
 import replay
 from helpers import gpu_ops
 from atom_amd.engine.core import StepEntry
-from atom_amd.kernels.hip import AttentionMeta
+from atom_amd.kernels.hip import AttentionMeta, QueryTurn
 
 pytestmark = pytest.mark.gpu
 DEV = "cuda:0"
@@ -108,7 +108,7 @@ def test_latent_prepare(dtype, heads, dim, rot, rank, dims, scaling):
 
     ops = gpu_ops()
     T, pre = 9, 5
-    ld = pre + heads * (dim + rot) + rank + rot + 3
+    ld = pre + heads * (dim + rot) + rank + rot + 4
     proj = rnd((T, ld), 1)
     positions = torch.tensor([0, 1, 2, 700, 701, 40000, 15, 16, 17])
     rope = ScaledRotary(dims, 5000.0, **(scaling or {}))
@@ -120,11 +120,22 @@ def test_latent_prepare(dtype, heads, dim, rot, rank, dims, scaling):
     pages = torch.zeros((3, 4, rank + rot), dtype=dtype, device=DEV)
     q_abs = torch.zeros((T, heads, rank + rot), dtype=dtype, device=DEV)
     kv_off = pre + heads * (dim + rot)
-    ops.latent_prepare(proj.to(DEV), pre, kv_off, heads, dim, rot, rank, dims, w.to(DEV), 1e-5, rope.freq, rope.mult,
-                       positions.int().to(DEV), slots.int().to(DEV), pages, q_abs, 0.37)
+    where, dpos = proj.to(DEV), positions.int().to(DEV)
+    ops.latent_prepare(where, pages, slots.int().to(DEV), dpos, kv_off, rank, rot, w.to(DEV), 1e-5, rope.freq, dims, rope.mult)
+    # the queries' rotated parts go past the absorbing product, whatever kernel takes it
+    up = rnd((heads, rank, dim), 3, dim ** -0.5).to(dtype).to(DEV)
+    for rows in (T, 3):
+        q_abs.zero_()
+        ops.heads_gemm(where, pre, ld, dim + rot, up, q_abs, 0, heads * (rank + rot), rank + rot, heads, rows, rank, dim,
+                       alpha=0.37, turn=QueryTurn(pre + dim, rank, rot, dims, rope.freq, rope.mult, 0.37, dpos[:rows]))
+        p = proj.double()[:rows]
+        q = p[:, pre:kv_off].view(rows, heads, dim + rot)
+        close(q_abs[:rows, :, rank:], pl.rotate_pairs(q[..., dim:], positions[:rows], dims, 5000.0, scaling) * 0.37, dtype,
+              "rotated queries")
+        absorbed = torch.stack([q[:, h, :dim] @ up[h].double().cpu().T for h in range(heads)], 1) * 0.37
+        close(q_abs[:rows, :, :rank], absorbed, dtype, "absorbed queries")
+        assert float(q_abs[rows:].abs().max() if rows < T else 0) == 0
     p = proj.double()
-    q = p[:, pre:kv_off].view(T, heads, dim + rot)[..., dim:]
-    close(q_abs[..., rank:], pl.rotate_pairs(q, positions, dims, 5000.0, scaling) * 0.37, dtype, "rotated queries")
     c = pl.rms_unit(p[:, kv_off:kv_off + rank], 1e-5) * w.double()
     k = pl.rotate_pairs(p[:, kv_off + rank:kv_off + rank + rot], positions, dims, 5000.0, scaling)
     want = torch.zeros((12, rank + rot), dtype=torch.float64)
