@@ -360,6 +360,40 @@ def savidra_pair(size: str) -> tuple[dict, dict]:
     return savi, qwen
 
 
+# The Benolix side has four layers: attention over latents within a window, with latents of its own, then reading the
+# first layer's, twice; the first with a dense feed-forward, the others with routed experts of which some are
+# identities.  Its closest relative here is Lotorax: the same attention over latents without window, query latent,
+# shared rows and gates per entry, and routed experts without identities, clamps and weights that are renormalised.  The
+# Lotorax side has four such layers of the same sizes, a dense feed-forward in the first, experts in the others.
+
+def benolix_pair(size: str) -> tuple[dict, dict]:
+    width, heads, rank, q_rank, ff, experts, identity, expert_ff, top, vocab = {
+        "1k": (1024, 8, 256, 512, 2816, 16, 4, 704, 2, 32768),
+        "2k": (2048, 16, 512, 1024, 5632, 32, 8, 704, 4, 32768),
+        "4k": (4096, 32, 512, 1536, 11264, 64, 16, 1408, 4, 65536),
+    }[size]
+    sizes = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": rank, "scale": 192 ** -0.5,
+             "rot": {"base": 1000000.0, "dims": 64}}
+    own = {**sizes, "q_rank": q_rank, "mask": {"size": 1024}}
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff, "limit": 7.0},
+           "router": {"experts": experts, "identity": identity, "top": top, "scale": 2.5}}
+    layer = lambda mixer, mlp: {"type": "latent_attention", "mixer": mixer, "mlp": mlp}  # noqa: E731
+    beno = {"architecture": "Benolix", "vocab": vocab, "width": width, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-6},
+            "postln_alpha": 2.0, "max_position_embeddings": 40960,
+            "layers": [layer(own, dense), layer({**own, "kv_from": 0}, moe), layer(own, moe),
+                       layer({**own, "kv_from": 2}, moe)]}
+    plain_moe = {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": experts, "top": top}}
+    loto = {"architecture": "Lotorax", "vocab": vocab, "width": width, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-6},
+            "max_position_embeddings": 40960, "layers": [layer(sizes, dense)] + [layer(sizes, plain_moe)] * 3}
+    return beno, loto
+
+
+def run_benolix(args) -> dict:
+    """Prefill and decode throughput of Benolix and of Lotorax at equal size, one engine after the other."""
+    return run_design(args, "benolix", "Benolix", benolix_pair, args.benolix, beside="Lotorax")
+
+
 def run_savidra(args) -> dict:
     """Prefill and decode throughput of Savidra and of Qwen3 at equal size, one engine after the other."""
     return run_design(args, "savidra", "Savidra", savidra_pair, args.savidra)
@@ -380,19 +414,19 @@ def run_leduvik(args) -> dict:
     return run_design(args, "leduvik", "Leduvik", leduvik_pair, args.leduvik)
 
 
-def run_design(args, key: str, design: str, pair, sizes: str) -> dict:
+def run_design(args, key: str, design: str, pair, sizes: str, beside: str = "Qwen3") -> dict:
     import torch
 
     from atom_amd import LLMEngine, SamplingParams
     from atom_amd.config import model_config_from_dict
 
-    out = {"metric": f"prefill tok/s and decode tok/s of the {design} design beside Qwen3 at equal size (bf16)",
+    out = {"metric": f"prefill tok/s and decode tok/s of the {design} design beside {beside} at equal size (bf16)",
            "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup, "dtype": "bf16",
            "data": "synthetic: seeded uniform random token ids, seeded random N(0, 0.02) weights",
            "config": {"batch": args.batch, "context": args.context, "layers": 4}, "sizes": {}}
     for size in sizes.split(","):
         row = out["sizes"][size] = {}
-        for name, raw in zip((key, "qwen3"), pair(size)):
+        for name, raw in zip((key, beside.lower()), pair(size)):
             max_len = max(4096, 2 * args.context)
             llm = LLMEngine(f"{name}-{size}-random", model_config=model_config_from_dict(raw), load_dummy="random",
                             seed=5, dtype="bf16", max_model_len=max_len, kv_cache_block_size=16,
@@ -417,8 +451,8 @@ def run_design(args, key: str, design: str, pair, sizes: str) -> dict:
                          "decode_tok_s": round(args.batch * args.steps / elapsed, 1)}
             print(f"[bench] {size} {name}: {row[name]}", file=sys.stderr, flush=True)
             release(llm)
-        row["prefill_ratio"] = round(row[key]["prefill_tok_s"] / row["qwen3"]["prefill_tok_s"], 3)
-        row["decode_ratio"] = round(row[key]["decode_tok_s"] / row["qwen3"]["decode_tok_s"], 3)
+        row["prefill_ratio"] = round(row[key]["prefill_tok_s"] / row[beside.lower()]["prefill_tok_s"], 3)
+        row["decode_ratio"] = round(row[key]["decode_tok_s"] / row[beside.lower()]["decode_tok_s"], 3)
     first = out["sizes"][sizes.split(",")[0]][key]
     out.update(value=first["decode_tok_s"], ms_per_step=first["decode_ms_per_step"], higher_is_better=True,
                scaling="weak", vs_baseline=None)
@@ -682,6 +716,9 @@ def main() -> int:
     ap.add_argument("--savidra", type=str, default="", metavar="SIZE[,SIZE]",
                     help="the Savidra design beside Qwen3 at equal size (1k, 2k, 4k: the width): prefill of --context "
                          "tokens and decode at --batch, four layers each")
+    ap.add_argument("--benolix", type=str, default="", metavar="SIZE[,SIZE]",
+                    help="the Benolix design beside Lotorax at equal size (1k, 2k, 4k: the width): prefill of --context "
+                         "tokens and decode at --batch, four layers each")
     ap.add_argument("--budget", type=int, default=None,
                     help="the scheduler's token budget of a step (mixed: 512 + N by default, so that portions stay 512)")
     ap.add_argument("--temperature", type=float, default=0.0, help="of the decode steps' sampling (0: greedy)")
@@ -715,6 +752,9 @@ def main() -> int:
         return 0
     if args.savidra:
         print(json.dumps(run_savidra(args)), flush=True)
+        return 0
+    if args.benolix:
+        print(json.dumps(run_benolix(args)), flush=True)
         return 0
     args.shape = args.shape or "8b"
     line = run_shape(args)
