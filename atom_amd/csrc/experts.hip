@@ -16,7 +16,7 @@
 //
 // The last two read an expert's rows once per (token, choice): the form for steps of few tokens.  Every sum runs in a
 // fixed order over a token's own data, so a token's result does not depend on what else is in the batch.
-#include "common.h"
+#include "lds_loads.h"
 
 struct RouterRule {
   int softmax;        // scores: 0 sigmoid, 1 softmax over the token's logits
@@ -227,34 +227,56 @@ experts_down_kernel(const T* __restrict__ x, const T* __restrict__ act_in, const
   const int tid = threadIdx.x, wave = tid / kWave, lane = tid % kWave;
   for (int i = tid; i < top * ff; i += 256) as[i] = to_f32(act_in[(size_t)t * top * ff + i]);
   __syncthreads();
-  for (int c = 0; c < kExpCols / 4; ++c) {
-    const int col = blockIdx.y * kExpCols + wave * (kExpCols / 4) + c;
-    if (col >= width) break;
-    float total = 0.f;
-    for (int k = 0; k < top; ++k) {
-      const int e = ids[(size_t)t * top + k];
-      if (e >= experts) {
-        total += weights[(size_t)t * top + k] * to_f32(x[(size_t)t * width + col]);
-        continue;
-      }
-      const TW* wr = w + ((size_t)e * width + col) * ff;
-      float s = 0.f;
-      bool done = false;
-      if constexpr (sizeof(TW) == 2) {
-        if (ff % 8 == 0) {
-          for (int i = lane * 8; i < ff; i += kWave * 8) {
-            const ex_bf16x8 wv = *reinterpret_cast<const ex_bf16x8*>(wr + i);
+  // a wave's columns side by side: their rows of w are independent loads, and a column is summed over the lanes once,
+  // for all of its choices together
+  constexpr int C = kExpCols / 4;
+  const int col0 = blockIdx.y * kExpCols + wave * C;
+  float total[C];
 #pragma unroll
-            for (int e = 0; e < 8; ++e) s = fmaf(as[k * ff + i + e], static_cast<float>(wv[e]), s);
-          }
-          done = true;
-        }
+  for (int c = 0; c < C; ++c) total[c] = 0.f;
+  for (int k = 0; k < top; ++k) {
+    const int e = ids[(size_t)t * top + k];
+    const float share = weights[(size_t)t * top + k];
+    if (e >= experts) {   // an identity expert: lane c brings x for column c
+      if (lane < C && col0 + lane < width) {
+        const float v = share * to_f32(x[(size_t)t * width + col0 + lane]);
+#pragma unroll
+        for (int c = 0; c < C; ++c) total[c] += lane == c ? v : 0.f;
       }
-      if (!done)
-        for (int i = lane; i < ff; i += kWave) s = fmaf(as[k * ff + i], to_f32(wr[i]), s);
-      total += weights[(size_t)t * top + k] * wave_sum(s);
+      continue;
     }
-    if (lane == 0) y[(size_t)t * width + col] = from_f32<T>(total);
+    const TW* we = w + (size_t)e * width * ff;
+    const TW* row[C];
+#pragma unroll
+    for (int c = 0; c < C; ++c) row[c] = we + (size_t)(col0 + c < width ? col0 + c : width - 1) * ff;
+    bool done = false;
+    if constexpr (sizeof(TW) == 2) {
+      if (ff % 8 == 0) {
+        for (int i = lane * 8; i < ff; i += kWave * 8) {
+          ex_bf16x8 wv[C];
+#pragma unroll
+          for (int c = 0; c < C; ++c) wv[c] = *reinterpret_cast<const ex_bf16x8*>(row[c] + i);
+#pragma unroll
+          for (int j = 0; j < 8; ++j) {
+            const float a = share * as[k * ff + i + j];
+#pragma unroll
+            for (int c = 0; c < C; ++c) total[c] = fmaf(a, static_cast<float>(wv[c][j]), total[c]);
+          }
+        }
+        done = true;
+      }
+    }
+    if (!done)
+      for (int i = lane; i < ff; i += kWave) {
+        const float a = share * as[k * ff + i];
+#pragma unroll
+        for (int c = 0; c < C; ++c) total[c] = fmaf(a, to_f32(row[c][i]), total[c]);
+      }
+  }
+#pragma unroll
+  for (int c = 0; c < C; ++c) {
+    const float sum = wave_sum(total[c]);
+    if (lane == 0 && col0 + c < width) y[(size_t)t * width + col0 + c] = from_f32<T>(sum);
   }
 }
 
@@ -303,7 +325,7 @@ ATOM_EXPORT int atom_experts_down(const void* x, const void* act_in, const void*
 
 // ------------------------------------------------------------------ many tokens: pairs sorted by expert, grouped products
 //
-//   experts_sort      one block: counts the pairs of every expert, gives each expert whole tiles of 64 rows
+//   experts_sort      one block: counts the pairs of every expert, gives each expert whole tiles of 64 or 128 rows
 //                     (padded), and every pair its row.  tile_expert[tile] = expert or -1; row_pair[row] = pair or
 //                     -1; pair_row[pair] = row, or -1 for an identity expert's pair, which gets none.  Rows of one
 //                     expert come in no fixed order; a row's result does not depend on its place.
@@ -322,15 +344,15 @@ typedef __attribute__((ext_vector_type(4))) __bf16 bf16x4;
 constexpr int kTileRows = 64;
 
 __global__ void __launch_bounds__(1024)
-experts_sort_kernel(const int* __restrict__ ids, int pairs, int experts, int max_tiles, int* __restrict__ tile_expert,
-                    int* __restrict__ row_pair, int* __restrict__ pair_row) {
+experts_sort_kernel(const int* __restrict__ ids, int pairs, int experts, int max_tiles, int tile_rows,
+                    int* __restrict__ tile_expert, int* __restrict__ row_pair, int* __restrict__ pair_row) {
   extern __shared__ int sm[];   // counts [experts], first row of each expert [experts]
   int* counts = sm;
   int* first = sm + experts;
   const int tid = threadIdx.x;
   for (int e = tid; e < experts; e += 1024) counts[e] = 0;
   for (int i = tid; i < max_tiles; i += 1024) tile_expert[i] = -1;
-  for (int i = tid; i < max_tiles * kTileRows; i += 1024) row_pair[i] = -1;
+  for (int i = tid; i < max_tiles * tile_rows; i += 1024) row_pair[i] = -1;
   __syncthreads();
   for (int i = tid; i < pairs; i += 1024)
     if (ids[i] < experts) atomicAdd(&counts[ids[i]], 1);
@@ -338,8 +360,8 @@ experts_sort_kernel(const int* __restrict__ ids, int pairs, int experts, int max
   if (tid == 0) {
     int tile = 0;
     for (int e = 0; e < experts; ++e) {
-      first[e] = tile * kTileRows;
-      const int n = (counts[e] + kTileRows - 1) / kTileRows;
+      first[e] = tile * tile_rows;
+      const int n = (counts[e] + tile_rows - 1) / tile_rows;
       for (int j = 0; j < n; ++j) tile_expert[tile + j] = e;
       tile += n;
       counts[e] = 0;   // now the fill level
@@ -494,30 +516,170 @@ grouped_down_kernel(const bf16_t* __restrict__ act_in, const bf16_t* __restrict_
   }
 }
 
-__global__ void experts_combine_kernel(const float* __restrict__ y, const bf16_t* __restrict__ x,
-                                       const int* __restrict__ pair_row, const float* __restrict__ weights,
-                                       bf16_t* __restrict__ out, int top, int width) {
-  const size_t t = blockIdx.x;
-  for (int c = threadIdx.x; c < width; c += blockDim.x) {
-    float total = 0.f;
-    for (int k = 0; k < top; ++k) {
-      const int row = pair_row[t * top + k];
-      total += weights[t * top + k] * (row >= 0 ? y[(size_t)row * width + c] : to_f32(x[t * width + c]));
+// The grouped products for experts with many rows: tiles of 128 rows x 128 rows of w (for gate and up 64 of each), K in
+// steps of 64.  Both operands are staged in LDS by loads that go there directly, one step ahead (two buffers, two blocks
+// a CU); a row's eight 16-byte pieces are permuted by its number, so that the operand reads of 16 rows at one place in K
+// fall on different banks.  Blocks that share an expert's rows of w and tiles of x sit on one XCD.
+// GATED: x rows are tokens (row_pair), act[row] = f(gate, up) in bfloat16; otherwise x rows are the tile's own (act) and
+// y[row] is float32.  Needs K % 64 = 0 and cols % 4 = 0.
+
+constexpr int kWideRows = 128;
+
+template <bool GATED>
+__global__ void __launch_bounds__(256, 2)
+grouped_wide_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, const int* __restrict__ tile_expert,
+                    const int* __restrict__ row_pair, bf16_t* __restrict__ act_out, float* __restrict__ y, int top,
+                    int cols, int k_size, int col_tiles, int tiles, ExpertGate f) {
+  __shared__ __attribute__((aligned(16))) unsigned char lds[2][2 * kWideRows * 128];
+  // tiles in runs of whole rows of the grid per XCD (consecutive blocks go to the eight XCDs in turn)
+  const int per = (int)(gridDim.x / 8);
+  const int id = (int)(blockIdx.x % 8) * per + (int)(blockIdx.x / 8);
+  const int tile = id / col_tiles, col_tile = id % col_tiles;
+  if (tile >= tiles) return;
+  const int e = tile_expert[tile];
+  if (e < 0) return;
+  const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid / kWave), lane = tid % kWave;
+  const int r = lane % 16, g = lane / 16;
+  const int wm = wave / 2, wn = wave % 2;
+  const int row0 = tile * kWideRows;
+  const bf16_t* we = w + (size_t)e * (GATED ? 2 : 1) * cols * k_size;
+  // staging: instruction j of a wave brings eight rows of x (and of w); the lane's piece of its row
+  const bf16_t* xsrc[4];
+  const bf16_t* wsrc[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int n = (wave * 4 + j) * 8 + lane / 8;   // 0 .. 127
+    const int piece = (lane % 8) ^ (n & 7);
+    size_t src_row = (size_t)(row0 + n);
+    if (GATED) {
+      const int pair = row_pair[row0 + n];
+      src_row = (size_t)(pair >= 0 ? pair / top : 0);
     }
-    out[t * width + c] = static_cast<bf16_t>(total);
+    xsrc[j] = x + src_row * k_size + piece * 8;
+    size_t wrow;
+    if (GATED) {   // rows of w by wave column: 32 gate rows, then the 32 up rows of the same columns
+      int c = col_tile * 64 + (n / 64) * 32 + n % 32;
+      c = c < cols ? c : cols - 1;
+      wrow = (size_t)((n / 32) % 2 ? cols + c : c);
+    } else {
+      int c = col_tile * 128 + n;
+      wrow = (size_t)(c < cols ? c : cols - 1);
+    }
+    wsrc[j] = we + wrow * k_size + piece * 8;
+  }
+  const unsigned base = lds_address(lds) + wave * 4 * 1024;
+  auto stage = [&](int buffer) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      load_to_lds(xsrc[j], base + buffer * (2 * kWideRows * 128) + j * 1024);
+      load_to_lds(wsrc[j], base + buffer * (2 * kWideRows * 128) + kWideRows * 128 + j * 1024);
+      xsrc[j] += 64;
+      wsrc[j] += 64;
+    }
+  };
+  f32x4 acc[4][4];   // [16 rows of w][16 rows of x]
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const int steps = k_size / 64;
+  arrived();
+  stage(0);
+  for (int s = 0; s < steps; ++s) {
+    arrived();
+    lds_barrier();
+    if (s + 1 < steps) stage((s + 1) & 1);
+    const unsigned char* xl = lds[s & 1] + (wm * 64 + r) * 128;
+    const unsigned char* wl = lds[s & 1] + kWideRows * 128 + (wn * 64 + r) * 128;
+#pragma unroll
+    for (int h = 0; h < 2; ++h) {
+      const int at = ((h * 4 + g) ^ (r & 7)) * 16;
+      bf16x8 xb[4], wa[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        xb[i] = *reinterpret_cast<const bf16x8*>(xl + i * 16 * 128 + at);
+        wa[i] = *reinterpret_cast<const bf16x8*>(wl + i * 16 * 128 + at);
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wa[i], xb[j], acc[i][j], 0, 0, 0);
+    }
+  }
+  // lane (r, g) holds rows 16 i + 4g .. + 3 of w for row 16 j + r of x
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const size_t row = (size_t)(row0 + wm * 64 + j * 16 + r);
+    if (GATED) {
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const int col = col_tile * 64 + wn * 32 + i * 16 + 4 * g;
+        bf16x4 o;
+#pragma unroll
+        for (int q = 0; q < 4; ++q) o[q] = static_cast<__bf16>(expert_gate(acc[i][j][q], acc[2 + i][j][q], f));
+        if (col < cols) *reinterpret_cast<bf16x4*>(act_out + row * cols + col) = o;
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int col = col_tile * 128 + wn * 64 + i * 16 + 4 * g;
+        if (col < cols) *reinterpret_cast<f32x4*>(y + row * cols + col) = acc[i][j];
+      }
+    }
   }
 }
 
-// Rows of the padded, sorted layout for `pairs` pairs over `experts` experts (an upper bound, in whole tiles).
-ATOM_EXPORT int atom_experts_grouped_tiles(int pairs, int experts) { return pairs / kTileRows + experts; }
+// out[t] from a token's rows of y and, for its identity experts, x: four columns a thread
+__global__ void __launch_bounds__(256)
+experts_combine4_kernel(const float* __restrict__ y, const bf16_t* __restrict__ x, const int* __restrict__ pair_row,
+                        const float* __restrict__ weights, bf16_t* __restrict__ out, int top, int width) {
+  const size_t t = blockIdx.x;
+  for (int c = threadIdx.x * 4; c < width; c += 1024) {
+    f32x4 total = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int k = 0; k < top; ++k) {
+      const int row = pair_row[t * top + k];
+      const float share = weights[t * top + k];
+      f32x4 v;
+      if (row >= 0) {
+        v = *reinterpret_cast<const f32x4*>(y + (size_t)row * width + c);
+      } else {
+        const bf16x4 b = *reinterpret_cast<const bf16x4*>(x + t * width + c);
+#pragma unroll
+        for (int q = 0; q < 4; ++q) v[q] = static_cast<float>(b[q]);
+      }
+      total += share * v;
+    }
+    bf16x4 o;
+#pragma unroll
+    for (int q = 0; q < 4; ++q) o[q] = static_cast<__bf16>(total[q]);
+    *reinterpret_cast<bf16x4*>(out + t * width + c) = o;
+  }
+}
+
+// Rows of the padded, sorted layout for `pairs` pairs over `experts` experts, and the rows of a tile: 128 where the
+// experts have that many on average or near it and the sizes suit the wide kernel, else 64.
+static int grouped_tile_rows(int pairs, int experts, int ff, int width) {
+  return pairs >= 64 * experts && ff % 64 == 0 && width % 64 == 0 ? kWideRows : kTileRows;
+}
+
+ATOM_EXPORT int atom_experts_grouped_rows(int pairs, int experts, int ff, int width) {
+  const int rows = grouped_tile_rows(pairs, experts, ff, width);
+  return (pairs / rows + experts) * rows;
+}
+
+// How many tiles that is at most.
+ATOM_EXPORT int atom_experts_grouped_tiles(int pairs, int experts, int ff, int width) {
+  return pairs / grouped_tile_rows(pairs, experts, ff, width) + experts;
+}
 
 ATOM_EXPORT int atom_experts_grouped_supports(int ff, int width, int experts) {
   return ff > 0 && width > 0 && ff % 8 == 0 && width % 8 == 0 && experts > 0 && experts <= 4096;
 }
 
 // x [tokens, width] bf16; gate_up [experts, 2 ff, width]; down [experts, width, ff]; ids, weights [tokens, top];
-// scratch: tile_expert [tiles], row_pair [tiles * 64], pair_row [tokens * top] (int32), act [tiles * 64, ff] bf16
-// (rows of padding are never read for a live row), y [tiles * 64, width] float32; out [tokens, width] bf16.
+// scratch: tile_expert [tiles], row_pair [rows], pair_row [tokens * top] (int32), act [rows, ff] bf16 (rows of padding
+// are never read for a live row), y [rows, width] float32; out [tokens, width] bf16.
 ATOM_EXPORT int atom_experts_grouped(const void* x, const void* gate_up, const void* down, const int* ids,
                                      const float* weights, int* tile_expert, int* row_pair, int* pair_row, void* act_buf,
                                      float* y, void* out, int tokens, int top, int experts, int ff, int width, int act,
@@ -527,15 +689,28 @@ ATOM_EXPORT int atom_experts_grouped(const void* x, const void* gate_up, const v
   if (!atom_experts_grouped_supports(ff, width, experts)) return ATOM_UNSUPPORTED;
   if (tokens == 0) return ATOM_OK;
   const int pairs = tokens * top;
-  const int tiles = atom_experts_grouped_tiles(pairs, experts);
-  if (tiles > 0x7fffffff / kTileRows) return ATOM_TOO_LARGE;
+  const int tile_rows = grouped_tile_rows(pairs, experts, ff, width);
+  const int tiles = atom_experts_grouped_tiles(pairs, experts, ff, width);
+  if (tiles > 0x7fffffff / kWideRows) return ATOM_TOO_LARGE;
   hipLaunchKernelGGL(experts_sort_kernel, dim3(1), dim3(1024), 2 * experts * sizeof(int), stream, ids, pairs, experts,
-                     tiles, tile_expert, row_pair, pair_row);
-  hipLaunchKernelGGL(grouped_gate_up_kernel, dim3(tiles, (ff + 63) / 64), dim3(256), 0, stream, (const bf16_t*)x,
-                     (const bf16_t*)gate_up, tile_expert, row_pair, (bf16_t*)act_buf, top, ff, width, f);
-  hipLaunchKernelGGL(grouped_down_kernel, dim3(tiles, (width + 127) / 128), dim3(256), 0, stream, (const bf16_t*)act_buf,
-                     (const bf16_t*)down, tile_expert, y, ff, width);
-  hipLaunchKernelGGL(experts_combine_kernel, dim3(tokens), dim3(256), 0, stream, y, (const bf16_t*)x, pair_row, weights,
+                     tiles, tile_rows, tile_expert, row_pair, pair_row);
+  if (tile_rows == kWideRows) {
+    const int up_tiles = (ff + 63) / 64, down_tiles = (width + 127) / 128;
+    const long up_blocks = ((long)tiles * up_tiles + 7) / 8 * 8, down_blocks = ((long)tiles * down_tiles + 7) / 8 * 8;
+    if (up_blocks > 0x7fffffffL / 256 || down_blocks > 0x7fffffffL / 256) return ATOM_TOO_LARGE;
+    hipLaunchKernelGGL((grouped_wide_kernel<true>), dim3((unsigned)up_blocks), dim3(256), 0, stream, (const bf16_t*)x,
+                       (const bf16_t*)gate_up, tile_expert, row_pair, (bf16_t*)act_buf, (float*)nullptr, top, ff, width,
+                       up_tiles, tiles, f);
+    hipLaunchKernelGGL((grouped_wide_kernel<false>), dim3((unsigned)down_blocks), dim3(256), 0, stream,
+                       (const bf16_t*)act_buf, (const bf16_t*)down, tile_expert, row_pair, (bf16_t*)nullptr, y, top, width, ff,
+                       down_tiles, tiles, f);
+  } else {
+    hipLaunchKernelGGL(grouped_gate_up_kernel, dim3(tiles, (ff + 63) / 64), dim3(256), 0, stream, (const bf16_t*)x,
+                       (const bf16_t*)gate_up, tile_expert, row_pair, (bf16_t*)act_buf, top, ff, width, f);
+    hipLaunchKernelGGL(grouped_down_kernel, dim3(tiles, (width + 127) / 128), dim3(256), 0, stream, (const bf16_t*)act_buf,
+                       (const bf16_t*)down, tile_expert, y, ff, width);
+  }
+  hipLaunchKernelGGL(experts_combine4_kernel, dim3(tokens), dim3(256), 0, stream, y, (const bf16_t*)x, pair_row, weights,
                      (bf16_t*)out, top, width);
   return launch_status();
 }

@@ -532,6 +532,135 @@ heads_gemm_mfma_kernel(const TX* __restrict__ x, long ldx, long hsx, const bf16_
   }
 }
 
+// For many rows: a block of 2 x 2 waves owns 128 tokens x 128 columns, a wave 64 x 64 of them, so that a 16-byte piece
+// read feeds four products; the next step's pieces are asked for before this one's products.  `vec`: y, its strides and the
+// gate's suit four columns at a time (n % 4 = 0).
+template <typename TX>
+struct HeadPieces;
+template <>
+struct HeadPieces<bf16_t> {
+  hg_bf16x8 v;
+  __device__ __forceinline__ void load(const bf16_t* p) { v = *reinterpret_cast<const hg_bf16x8*>(p); }
+  __device__ __forceinline__ hg_bf16x8 get(bool ok) const {
+    const hg_bf16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
+    return ok ? v : zero;
+  }
+};
+template <>
+struct HeadPieces<float> {
+  hg_f32x4 a, b;
+  __device__ __forceinline__ void load(const float* p) {
+    a = *reinterpret_cast<const hg_f32x4*>(p);
+    b = *reinterpret_cast<const hg_f32x4*>(p + 4);
+  }
+  __device__ __forceinline__ hg_bf16x8 get(bool ok) const {
+    hg_bf16x8 out;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      out[i] = static_cast<__bf16>(ok ? a[i] : 0.f);
+      out[4 + i] = static_cast<__bf16>(ok ? b[i] : 0.f);
+    }
+    return out;
+  }
+};
+
+template <typename TX, typename TY>
+__global__ void __launch_bounds__(256, 2)
+heads_gemm_wide_kernel(const TX* __restrict__ x, long ldx, long hsx, const bf16_t* __restrict__ w, TY* __restrict__ y,
+                       long ldy, long hsy, ProductGate gate, QueryTurn turn, int m, int n, int k, float alpha, int vec) {
+  const int tid = threadIdx.x, wave = tid / kWave, lane = tid % kWave, r = lane % 16, g = lane / 16;
+  const int h = blockIdx.z;
+  if ((int)blockIdx.x * 128 >= n) {   // the column of blocks behind the product's
+    const int t0 = (int)blockIdx.y * 128;
+    turn_queries<TY>(turn, h, t0, m - t0 < 128 ? m - t0 : 128);
+    return;
+  }
+  const int row0 = blockIdx.y * 128 + (wave / 2) * 64;
+  const int col0 = blockIdx.x * 128 + (wave % 2) * 64;
+  // rows and columns beyond the product's are read as its last ones and not written
+  const TX* xrow[4];
+  const bf16_t* wrow[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int row = row0 + i * 16 + r < m ? row0 + i * 16 + r : m - 1;
+    const int col = col0 + i * 16 + r < n ? col0 + i * 16 + r : n - 1;
+    xrow[i] = x + (size_t)row * ldx + (size_t)h * hsx;
+    wrow[i] = w + ((size_t)h * n + col) * k;
+  }
+  hg_f32x4 acc[4][4];   // [16 columns][16 rows]
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = hg_f32x4{0.f, 0.f, 0.f, 0.f};
+  HeadPieces<TX> xp[2][4];
+  HeadPieces<bf16_t> wp[2][4];
+  auto fetch = [&](int buffer, int k0) {
+    const int kk = k0 + 8 * g < k ? k0 + 8 * g : k - 8;   // past the end: the last piece, which counts as zeros
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      xp[buffer][i].load(xrow[i] + kk);
+      wp[buffer][i].load(wrow[i] + kk);
+    }
+  };
+  auto multiply = [&](int buffer, int k0) {
+    const bool ok = k0 + 8 * g < k;
+    hg_bf16x8 xb[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) xb[j] = xp[buffer][j].get(ok);
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wp[buffer][i].get(true), xb[j], acc[i][j], 0, 0, 0);
+  };
+  fetch(0, 0);
+  for (int k0 = 0; k0 < k; k0 += 64) {
+    fetch(1, k0 + 32);
+    multiply(0, k0);
+    fetch(0, k0 + 64);
+    multiply(1, k0 + 32);
+  }
+  // lane (r, g) holds columns col0 + 16 i + 4g .. + 3 of row row0 + 16 j + r
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int row = row0 + j * 16 + r;
+    if (row >= m) continue;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int col = col0 + i * 16 + 4 * g;
+      if (col >= n) continue;
+      TY* dst = y + (size_t)row * ldy + (size_t)h * hsy + col;
+      hg_f32x4 v = acc[i][j] * alpha;
+      if (vec) {
+        if (gate.g) {
+          if (gate.csg) {
+            const hg_f32x4 gv = *reinterpret_cast<const hg_f32x4*>(gate.g + row * gate.ldg + (size_t)h * gate.hsg + col);
+#pragma unroll
+            for (int q = 0; q < 4; ++q) v[q] *= 1.f / (1.f + expf(-gv[q]));
+          } else {
+            v *= gate_value(gate, row, h, 0);
+          }
+        }
+        if constexpr (sizeof(TY) == 2) {
+          typedef __attribute__((ext_vector_type(4))) __bf16 hg_bf16x4;
+          hg_bf16x4 o;
+#pragma unroll
+          for (int q = 0; q < 4; ++q) o[q] = static_cast<__bf16>(v[q]);
+          *reinterpret_cast<hg_bf16x4*>(dst) = o;
+        } else {
+          *reinterpret_cast<hg_f32x4*>(dst) = v;
+        }
+      } else {
+#pragma unroll
+        for (int q = 0; q < 4; ++q)
+          if (col + q < n) dst[q] = from_f32<TY>(v[q] * (gate.g ? gate_value(gate, row, h, col + q) : 1.f));
+      }
+    }
+  }
+}
+
+constexpr int kHWideRows = 96;   // from here on the wide tiles
+
 ATOM_EXPORT int atom_heads_gemm_mfma_supports(int x_dtype, int w_dtype, long x_offset, long ldx, long hsx, int k) {
   if (w_dtype != ATOM_BF16 || k % 8) return 0;
   const long unit = x_dtype == ATOM_BF16 ? 8 : 4;   // elements of 16 bytes
@@ -558,6 +687,24 @@ ATOM_EXPORT int atom_heads_gemm_mfma(const void* x, int x_dtype, long ldx, long 
 #define LAUNCH(TX, TY, SPLIT)                                                                                       \
   hipLaunchKernelGGL((heads_gemm_mfma_kernel<TX, TY, SPLIT>), grid, block, 0, stream, (const TX*)x, ldx, hsx,      \
                      (const bf16_t*)w, (TY*)y, ldy, hsy, g, q, m, n, k, alpha)
+  if (!split && m >= kHWideRows) {
+    const long unit = 4;   // entries that are read or written together
+    const size_t y_align = (y_dtype == ATOM_BF16 ? 2 : 4) * unit;
+    const int vec = n % unit == 0 && ldy % unit == 0 && hsy % unit == 0 && (size_t)y % y_align == 0 &&
+                    (g.g == nullptr || g.csg == 0 || ((size_t)g.g % 16 == 0 && g.ldg % unit == 0 && g.hsg % unit == 0));
+    grid = dim3((n + 127) / 128 + (rot > 0 ? 1 : 0), (m + 127) / 128, heads);
+#define WIDE(TX, TY)                                                                                                \
+  hipLaunchKernelGGL((heads_gemm_wide_kernel<TX, TY>), grid, block, 0, stream, (const TX*)x, ldx, hsx, (const bf16_t*)w, \
+                     (TY*)y, ldy, hsy, g, q, m, n, k, alpha, vec)
+    switch (x_dtype * 2 + y_dtype) {
+      case 0: WIDE(float, float); break;
+      case 1: WIDE(float, bf16_t); break;
+      case 2: WIDE(bf16_t, float); break;
+      default: WIDE(bf16_t, bf16_t); break;
+    }
+#undef WIDE
+    return launch_status();
+  }
   if (split) {
     if (y_dtype == ATOM_F32) LAUNCH(float, float, true);
     else LAUNCH(float, bf16_t, true);

@@ -298,29 +298,48 @@ __global__ void __launch_bounds__(256) latent_mfma_kernel(LatentParams p) {
   }
 }
 
-// out[row] = sum_p o_p exp(m_p - M) / (sum_p l_p exp(m_p - M) + exp(sink - M)), M the largest of the m_p and the sink
+// out[row] = sum_p o_p exp(m_p - M) / (sum_p l_p exp(m_p - M) + exp(sink - M)), M the largest of the m_p and the sink.
+// A block of 128 threads a row, four entries a thread, four parts' loads in flight; rank % 4 = 0.
 __global__ void __launch_bounds__(128)
 latent_merge_kernel(const float* __restrict__ ws_o, const float* __restrict__ ws_ml, const float* __restrict__ sink,
                     bf16_t* __restrict__ out, int heads, int rank, int parts) {
   __shared__ float share[64];   // the parts' weights exp(m_p - M) / denominator
-  __shared__ float scratch[16];
   const size_t row = blockIdx.x;
   const int head = (int)(row % heads);
   const int tid = threadIdx.x;
   const float* ml = ws_ml + row * parts * 2;
-  const float sk = sink ? sink[head] : -INFINITY;
-  const float mine = tid < parts ? ml[2 * tid] : -INFINITY;
-  const float top = fmaxf(block_max(mine, scratch), sk);
-  const float w = (tid < parts && mine != -INFINITY) ? __expf(mine - top) : 0.f;
-  float denom = block_sum(tid < parts ? w * ml[2 * tid + 1] : 0.f, scratch);
-  if (sink && top != -INFINITY) denom += __expf(sk - top);
-  if (tid < parts) share[tid] = denom > 0.f ? w / denom : 0.f;
-  __syncthreads();
-  for (int e = tid; e < rank; e += 128) {
-    float a = 0.f;
-    for (int q = 0; q < parts; ++q) a += ws_o[(row * parts + q) * rank + e] * share[q];
-    out[row * rank + e] = static_cast<bf16_t>(a);
+  if (tid < kWave) {            // one wave holds all parts (64 at most)
+    const float sk = sink ? sink[head] : -INFINITY;
+    const float mine = tid < parts ? ml[2 * tid] : -INFINITY;
+    const float sum = tid < parts ? ml[2 * tid + 1] : 0.f;
+    const float top = fmaxf(wave_max(mine), sk);
+    const float w = mine != -INFINITY ? __expf(mine - top) : 0.f;
+    float denom = wave_sum(w * sum);
+    if (sink && top != -INFINITY) denom += __expf(sk - top);
+    share[tid] = denom > 0.f ? w / denom : 0.f;
   }
+  __syncthreads();
+  for (int e = tid * 4; e < rank; e += 512) {
+    const float* src = ws_o + row * parts * rank + e;
+    f32x4 a = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int q = 0; q < parts; ++q) a += *reinterpret_cast<const f32x4*>(src + (size_t)q * rank) * share[q];
+    bf16x4 o;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o[i] = static_cast<__bf16>(a[i]);
+    *reinterpret_cast<bf16x4*>(out + row * rank + e) = o;
+  }
+}
+
+ATOM_EXPORT int atom_latent_merge(const float* ws_o, const float* ws_ml, const float* sink, void* out, int rows, int heads,
+                                  int rank, int parts, hipStream_t stream) {
+  if (rows < 0 || heads <= 0 || rank <= 0 || (rank % 4) || parts < 1) return ATOM_BAD_SHAPE;
+  if (parts > 64) return ATOM_TOO_LARGE;
+  if (ws_o == nullptr || ws_ml == nullptr || out == nullptr) return ATOM_BAD_SHAPE;
+  if (rows == 0) return ATOM_OK;
+  hipLaunchKernelGGL(latent_merge_kernel, dim3(rows), dim3(128), 0, stream, ws_o, ws_ml, sink, (bf16_t*)out, heads, rank,
+                     parts);
+  return launch_status();
 }
 
 // The register sets the kernel is built for: (rank up to 16 RT, width up to 32 KS).
@@ -395,9 +414,6 @@ ATOM_EXPORT int atom_latent_attention_mfma(const void* q, const void* pages, voi
   else LAUNCH(32, 18);
 #undef LAUNCH
   if (hipGetLastError() != hipSuccess) return ATOM_LAUNCH_FAILED;
-  if (parts > 1) {
-    hipLaunchKernelGGL(latent_merge_kernel, dim3(tokens * heads), dim3(128), 0, stream, ws_o, ws_ml, sink,
-                       (bf16_t*)out, heads, rank, parts);
-  }
+  if (parts > 1) return atom_latent_merge(ws_o, ws_ml, sink, out, tokens * heads, heads, rank, parts, stream);
   return launch_status();
 }

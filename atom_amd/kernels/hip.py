@@ -208,8 +208,10 @@ class HipKernels:
                    "atom_layernorm", "atom_embedding_scaled", "atom_sum_concat", "atom_gated_act", "atom_latent_prepare",
                    "atom_heads_gemm", "atom_latent_attention", "atom_conv_silu_state", "atom_delta_rule",
                    "atom_delta_out", "atom_router_choose", "atom_experts_gate_up", "atom_experts_down",
+                   "atom_latent_attention_tile", "atom_latent_tile_supports", "atom_latent_merge",
                    "atom_latent_attention_mfma", "atom_latent_mfma_supports", "atom_latent_mfma_tokens_per_tile",
-                   "atom_experts_grouped", "atom_experts_grouped_tiles", "atom_experts_grouped_supports",
+                   "atom_experts_grouped", "atom_experts_grouped_tiles", "atom_experts_grouped_rows",
+                   "atom_experts_grouped_supports",
                    "atom_heads_gemm_mfma", "atom_heads_gemm_mfma_supports", "atom_rmsnorm_post", "atom_rmsnorm_rows",
                    "atom_cast_rows", "atom_token_gate", "atom_embedding_bigram", "atom_rglru_scan",
                    "atom_keys_as_values_write", "atom_sigmoid_gate", "atom_bias_rows", "atom_linear_scan", "atom_token_shift",
@@ -243,6 +245,7 @@ class HipKernels:
         self.use_fused_decode = True    # decode-only steps of few rows: norm, rotation and cache write inside attention
         self.use_together_tiles = True  # attention with the heads together on the matrix cores, for prompt portions
         self.use_mfma_latent = True     # attention over latent pages on the matrix cores (bfloat16, sizes it is built for)
+        self.use_latent_tiles = True    # ... its form for a latent of 128, 256 or 512 entries and 64 rotated ones
         # routed experts: from this many (token, choice) pairs on, the pairs are sorted by expert and run as grouped
         # products on the matrix cores; below, every pair reads its expert's rows itself
         self.grouped_experts_from = 64
@@ -1129,15 +1132,19 @@ class HipKernels:
             self._stream()))
         return y
 
-    def latent_parts(self, meta: AttentionMeta, heads: int, window: int | None) -> int:
-        """Over how many blocks a row's keys are split in the matrix-core kernel: one for steps with prompt
-        portions (their tiles fill the chip); for single tokens enough blocks to fill it twice, 128 keys each at
-        least."""
+    def latent_parts(self, meta: AttentionMeta, heads: int, window: int | None, tiles: bool = False) -> int:
+        """Over how many blocks a row's keys are split in the matrix-core kernels: one for steps with prompt portions
+        (their tiles fill the chip); for single tokens enough blocks to fill it twice, or half of it with the tile kernel
+        (``tiles``), whose blocks have a CU to themselves; 64 keys each at least."""
         if meta.max_q_len > 1:
             return 1
         blocks = max(1, meta.num_seqs * -(-heads // 64))
         visible = min(meta.max_context_len, window) if window else meta.max_context_len
-        return max(1, min(-(-2 * self.num_cus // blocks), -(-visible // 128), 64))
+        if tiles:
+            # 8 requests of 16 heads at 2,064 keys: 28.5 / 20.7 / 17.4 / 24.9 us with 4 / 8 / 16 / 32 parts: beyond half
+            # the chip's CUs the results to merge cost more than the shorter walks save
+            return max(1, min(-(-self.num_cus // (2 * blocks)), -(-visible // 64), 32))
+        return max(1, min(-(-2 * self.num_cus // blocks), -(-visible // 64), 64))
 
     def latent_attention(self, q_abs, pages, out, meta: AttentionMeta, rank: int, sink=None, window: int | None = None,
                          parts: int | None = None):
@@ -1163,12 +1170,23 @@ class HipKernels:
             self._check("context_lens", meta.context_lens, torch.int32, (meta.num_seqs,))
             if meta.block_tables.shape[0] != meta.num_seqs:
                 raise KernelError("attention: one block table row per request is needed")
+            tiles = bool(self.use_latent_tiles and self.lib.atom_latent_tile_supports(rank, width))
             if parts is None:
-                parts = self.latent_parts(meta, heads, window)
+                parts = self.latent_parts(meta, heads, window, tiles)
             ws_o = ws_ml = None
             if parts > 1:
                 ws_o = self.workspace("latent_o", tokens * heads * parts * rank)
                 ws_ml = self.workspace("latent_ml", tokens * heads * parts * 2)
+            if tiles:
+                self._done("latent_attention_tile", self.lib.atom_latent_attention_tile(
+                    _ptr(q_abs), _ptr(pages), _ptr(out), _ptr(ws_o), _ptr(ws_ml), _ptr(meta.cu_seqlens_q),
+                    _ptr(meta.context_lens), _ptr(meta.block_tables), meta.block_tables.shape[1], _ptr(sink),
+                    meta.num_seqs, tokens, meta.max_q_len, heads, rank, width, meta.page_size, int(window or 0), parts,
+                    self._stream()))
+                if parts > 1:
+                    self._done("latent_merge", self.lib.atom_latent_merge(
+                        _ptr(ws_o), _ptr(ws_ml), _ptr(sink), _ptr(out), tokens * heads, heads, rank, parts, self._stream()))
+                return out
             self._done("latent_attention_mfma", self.lib.atom_latent_attention_mfma(
                 _ptr(q_abs), _ptr(pages), _ptr(out), _ptr(ws_o), _ptr(ws_ml), _ptr(meta.cu_seqlens_q),
                 _ptr(meta.context_lens), _ptr(meta.block_tables), meta.block_tables.shape[1], _ptr(sink), meta.num_seqs,
@@ -1869,15 +1887,16 @@ class HipKernels:
                 ctypes.c_float(slope), ctypes.c_float(shift)]
         if (x.dtype == torch.bfloat16 and gate_up.dtype == torch.bfloat16 and tokens * top >= self.grouped_experts_from
                 and self.lib.atom_experts_grouped_supports(ff, width, experts)):
-            tiles = self.lib.atom_experts_grouped_tiles(tokens * top, experts)
-            ints = self.workspace("experts_ints", tiles * 65 + tokens * top, torch.int32)
-            act = self.workspace("experts_act", tiles * 64 * ff, torch.bfloat16)
-            rows = self.workspace("experts_rows", tiles * 64 * width)
+            tiles = self.lib.atom_experts_grouped_tiles(tokens * top, experts, ff, width)
+            padded = self.lib.atom_experts_grouped_rows(tokens * top, experts, ff, width)
+            ints = self.workspace("experts_ints", tiles + padded + tokens * top, torch.int32)
+            act = self.workspace("experts_act", padded * ff, torch.bfloat16)
+            rows = self.workspace("experts_rows", padded * width)
             y = torch.empty((tokens, width), dtype=x.dtype, device=x.device)
             self._done("experts_grouped", self.lib.atom_experts_grouped(
                 _ptr(x), _ptr(gate_up), _ptr(down), _ptr(ids), _ptr(weights), _ptr(ints),
-                ctypes.c_void_p(ints.data_ptr() + 4 * tiles), ctypes.c_void_p(ints.data_ptr() + 4 * tiles * 65), _ptr(act),
-                _ptr(rows), _ptr(y), tokens, top, experts, ff, width, *gate, self._stream()))
+                ctypes.c_void_p(ints.data_ptr() + 4 * tiles), ctypes.c_void_p(ints.data_ptr() + 4 * (tiles + padded)),
+                _ptr(act), _ptr(rows), _ptr(y), tokens, top, experts, ff, width, *gate, self._stream()))
             return y
         act = torch.empty((tokens * top, ff), dtype=x.dtype, device=x.device)
         self._done("experts_gate_up", self.lib.atom_experts_gate_up(

@@ -79,7 +79,8 @@ def test_query_latent_and_key_rows(dtype, cq, rank, rot, dims):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("x_dtype", DTYPES)
 @pytest.mark.parametrize("H,m,n,k", [(3, 70, 21, 16), (2, 200, 100, 40), (5, 33, 64, 128), (3, 5, 24, 32), (4, 9, 7, 13),
-                                     (2, 3, 5, 13), (2, 130, 128, 512), (16, 8, 128, 512), (1, 1, 1, 1)])
+                                     (2, 3, 5, 13), (2, 130, 128, 512), (16, 8, 128, 512), (1, 1, 1, 1),
+                                     (3, 97, 132, 40), (2, 300, 256, 72), (1, 128, 20, 8), (2, 200, 130, 96)])
 def test_per_head_products_with_a_gate_per_entry(dtype, x_dtype, H, m, n, k):
     """Every kernel of the per-head product (few rows, tiles, matrix cores) with one gate value per output entry."""
     ops = gpu_ops()
@@ -102,7 +103,8 @@ def test_per_head_products_with_a_gate_per_entry(dtype, x_dtype, H, m, n, k):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("H,m,d,rot,dims,rank", [(3, 70, 8, 6, 4, 24), (16, 5, 128, 64, 64, 512), (5, 200, 16, 16, 16, 40),
-                                                 (2, 9, 13, 5, 2, 11), (4, 3, 7, 3, 0, 20), (3, 65, 32, 8, 8, 64)])
+                                                 (2, 9, 13, 5, 2, 11), (4, 3, 7, 3, 0, 20), (3, 65, 32, 8, 8, 64),
+                                                        (4, 150, 24, 8, 8, 200), (2, 257, 128, 64, 64, 512)])
 def test_absorbing_product_turns_the_rotated_parts(dtype, H, m, d, rot, dims, rank):
     ops = gpu_ops()
     width, ld = rank + rot, H * (d + rot)
@@ -128,7 +130,7 @@ def _attend(q_abs, rows, rank, pos, window):
 
 
 SIZES = [(32, 8, 3, 16), (64, 16, 16, 8), (20, 6, 5, 4), (128, 64, 20, 16), (256, 64, 8, 16), (512, 64, 16, 16), (48, 8, 70, 4),
-         (32, 16, 2, 5), (160, 32, 33, 32)]
+         (32, 16, 2, 5), (160, 32, 33, 32), (512, 64, 3, 7), (512, 64, 32, 16), (128, 64, 70, 4), (256, 64, 40, 8), (128, 64, 16, 16)]
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -240,7 +242,8 @@ def test_router_softmax_scores(outputs, top, scale):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("width,ff,experts,identity,top,tokens", [
     (48, 40, 5, 2, 2, 13), (40, 16, 6, 0, 3, 1), (64, 32, 8, 8, 1, 70), (48, 40, 2, 5, 4, 300), (136, 72, 33, 7, 4, 129),
-    (44, 18, 5, 2, 3, 50), (264, 88, 10, 3, 2, 64), (32, 24, 1, 1, 2, 8), (56, 36, 3, 1, 2, 90)])
+    (44, 18, 5, 2, 3, 50), (264, 88, 10, 3, 2, 64), (32, 24, 1, 1, 2, 8), (56, 36, 3, 1, 2, 90),
+    (128, 64, 3, 1, 2, 300), (192, 128, 5, 0, 3, 250), (64, 192, 2, 1, 2, 515), (320, 64, 9, 3, 4, 161)])
 def test_experts_with_clamped_gates_and_identities(dtype, width, ff, experts, identity, top, tokens):
     """Few and many (token, choice) pairs, sizes the grouped products take and not; gate and up rows reach the clamp;
     some tokens have identity experts only, some none."""
