@@ -36,41 +36,49 @@ latent_prepare_kernel(const float* __restrict__ proj, int ld, int cq_off, int cq
                       T* __restrict__ cq, int kv_off, int rank, int rot, int rot_dims, const float* __restrict__ norm_w,
                       float eps, const double* __restrict__ freq, float mult, const int* __restrict__ positions,
                       const int* __restrict__ slots, T* __restrict__ pages) {
-  __shared__ float scratch[16];
+  __shared__ float scratch[2][4];
   const int t = blockIdx.x;
   const int tid = threadIdx.x;
   const float* row = proj + (size_t)t * ld;
-  if (cq_rank > 0) {
-    float part = 0.f;
-    for (int i = tid; i < cq_rank; i += 256) {
-      const float v = row[cq_off + i];
-      part += v * v;
+  const int slot = slots ? slots[t] : -1;   // the same for the whole block
+  // both norms' sums of squares in one pass and one meeting of the waves
+  float ss_q = 0.f, ss_k = 0.f;
+#pragma unroll 4
+  for (int i = tid; i < cq_rank; i += 256) ss_q += row[cq_off + i] * row[cq_off + i];
+  if (slot >= 0) {
+#pragma unroll 4
+    for (int i = tid; i < rank; i += 256) ss_k += row[kv_off + i] * row[kv_off + i];
+    // the shared rotated key part: by the last wave first, while the others are still adding
+    T* dst = pages + (size_t)slot * (rank + rot) + rank;
+    for (int i = 255 - tid; i < rot; i += 256) {
+      float v = row[kv_off + rank + i];
+      if (i < rot_dims) {
+        float c, s;
+        pair_angle(positions[t], freq[i >> 1], mult, &c, &s);
+        const float other = row[kv_off + rank + (i ^ 1)];
+        v = (i & 1) ? v * c + other * s : v * c - other * s;
+      }
+      dst[i] = from_f32<T>(v);
     }
-    const float rstd = 1.f / sqrtf(block_sum(part, scratch) / (float)cq_rank + eps);
+  }
+  ss_q = wave_sum(ss_q);
+  ss_k = wave_sum(ss_k);
+  if (tid % kWave == 0) {
+    scratch[0][tid / kWave] = ss_q;
+    scratch[1][tid / kWave] = ss_k;
+  }
+  __syncthreads();
+  // x / sqrt(mean(x^2) + eps) * w
+  if (cq_rank > 0) {
+    const float rstd = 1.f / sqrtf((scratch[0][0] + scratch[0][1] + scratch[0][2] + scratch[0][3]) / (float)cq_rank + eps);
+#pragma unroll 4
     for (int i = tid; i < cq_rank; i += 256) cq[(size_t)t * cq_rank + i] = from_f32<T>(row[cq_off + i] * rstd * cq_w[i]);
   }
-  const int slot = slots ? slots[t] : -1;   // the same for the whole block
-  if (slot < 0) return;
-  const int pos = positions[t];
-  T* dst = pages + (size_t)slot * (rank + rot);
-  // the latent: x / sqrt(mean(x^2) + eps) * w
-  float part = 0.f;
-  for (int i = tid; i < rank; i += 256) {
-    const float v = row[kv_off + i];
-    part += v * v;
-  }
-  const float rstd = 1.f / sqrtf(block_sum(part, scratch) / (float)rank + eps);
-  for (int i = tid; i < rank; i += 256) dst[i] = from_f32<T>(row[kv_off + i] * rstd * norm_w[i]);
-  // the shared rotated key part
-  for (int i = tid; i < rot; i += 256) {
-    float v = row[kv_off + rank + i];
-    if (i < rot_dims) {
-      float c, s;
-      pair_angle(pos, freq[i >> 1], mult, &c, &s);
-      const float other = row[kv_off + rank + (i ^ 1)];
-      v = (i & 1) ? v * c + other * s : v * c - other * s;
-    }
-    dst[rank + i] = from_f32<T>(v);
+  if (slot >= 0) {
+    const float rstd = 1.f / sqrtf((scratch[1][0] + scratch[1][1] + scratch[1][2] + scratch[1][3]) / (float)rank + eps);
+    T* dst = pages + (size_t)slot * (rank + rot);
+#pragma unroll 4
+    for (int i = tid; i < rank; i += 256) dst[i] = from_f32<T>(row[kv_off + i] * rstd * norm_w[i]);
   }
 }
 
@@ -411,11 +419,12 @@ ATOM_EXPORT int atom_latent_attention(const void* q_abs, const void* pages, void
 
 // ------------------------------------------------------------------ the per-head products on the matrix cores
 //
-// The same product as heads_gemm with bfloat16 weights, for many rows: the head's weight rows are the A operand and
-// the tokens the B operand, both read straight from memory (a float32 input is rounded to bfloat16 on the way, or,
-// where the product is to be the float32 one, split into three bfloat16 pieces that are multiplied one by one), so a
-// lane ends up with four consecutive columns of one token.  A block of 2 x 2 waves owns 64 tokens x 64 columns.
-// Needs k % 8 == 0 and offsets and strides of x that keep its 8-element pieces aligned.
+// The same product as heads_gemm with bfloat16 weights: the head's weight rows are the A operand and the tokens the B
+// operand, both read straight from memory (a float32 input is rounded to bfloat16 on the way, or, where the product is
+// to be the float32 one, split into three bfloat16 pieces that are multiplied one by one), so a lane ends up with four
+// consecutive columns of one token.  Three kernels: the exact one (a block of 2 x 2 waves owns 64 tokens x 64 columns),
+// one for many rows and one for few.  All need k % 8 == 0 and offsets and strides of x that keep its 8-element pieces
+// aligned.
 
 typedef __attribute__((ext_vector_type(4))) float hg_f32x4;
 typedef __attribute__((ext_vector_type(8))) __bf16 hg_bf16x8;
@@ -423,19 +432,6 @@ typedef __attribute__((ext_vector_type(8))) __bf16 hg_bf16x8;
 __device__ __forceinline__ hg_bf16x8 hg_load8(const bf16_t* p, bool ok) {
   const hg_bf16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
   return ok ? *reinterpret_cast<const hg_bf16x8*>(p) : zero;
-}
-
-__device__ __forceinline__ hg_bf16x8 hg_load8(const float* p, bool ok) {
-  hg_bf16x8 out = {0, 0, 0, 0, 0, 0, 0, 0};
-  if (ok) {
-    const hg_f32x4 a = *reinterpret_cast<const hg_f32x4*>(p), b = *reinterpret_cast<const hg_f32x4*>(p + 4);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      out[i] = static_cast<__bf16>(a[i]);
-      out[4 + i] = static_cast<__bf16>(b[i]);
-    }
-  }
-  return out;
 }
 
 // A float32 input in three bfloat16 pieces, x = hi + mid + lo exactly (3 x 8 bits of mantissa): the products of each
@@ -460,9 +456,9 @@ __device__ __forceinline__ void hg_load8_split(const float* p, bool ok, hg_bf16x
   }
 }
 
-template <typename TX, typename TY, bool SPLIT = false>
+template <typename TY>
 __global__ void __launch_bounds__(256)
-heads_gemm_mfma_kernel(const TX* __restrict__ x, long ldx, long hsx, const bf16_t* __restrict__ w, TY* __restrict__ y,
+heads_gemm_split_kernel(const float* __restrict__ x, long ldx, long hsx, const bf16_t* __restrict__ w, TY* __restrict__ y,
                        long ldy, long hsy, ProductGate gate, QueryTurn turn, int m, int n, int k, float alpha) {
   const int tid = threadIdx.x, wave = tid / kWave, lane = tid % kWave, r = lane % 16, g = lane / 16;
   const int h = blockIdx.z;
@@ -472,7 +468,7 @@ heads_gemm_mfma_kernel(const TX* __restrict__ x, long ldx, long hsx, const bf16_
   }
   const int row0 = blockIdx.y * 64 + (wave / 2) * 32;
   const int col0 = blockIdx.x * 64 + (wave % 2) * 32;
-  const TX* xrow[2];
+  const float* xrow[2];
   bool rok[2];
 #pragma unroll
   for (int rt = 0; rt < 2; ++rt) {
@@ -496,23 +492,18 @@ heads_gemm_mfma_kernel(const TX* __restrict__ x, long ldx, long hsx, const bf16_
   for (int k0 = 0; k0 < k; k0 += 32) {
     const int kk = k0 + 8 * g;
     const bool kok = kk < k;
-    hg_bf16x8 xb[2], wa[2];
-    [[maybe_unused]] hg_bf16x8 xm[2], xl[2];
+    hg_bf16x8 xb[2], xm[2], xl[2], wa[2];
 #pragma unroll
-    for (int rt = 0; rt < 2; ++rt) {
-      if constexpr (SPLIT) hg_load8_split(xrow[rt] + kk, kok && rok[rt], &xb[rt], &xm[rt], &xl[rt]);
-      else xb[rt] = hg_load8(xrow[rt] + kk, kok && rok[rt]);
-    }
+    for (int rt = 0; rt < 2; ++rt) hg_load8_split(xrow[rt] + kk, kok && rok[rt], &xb[rt], &xm[rt], &xl[rt]);
 #pragma unroll
     for (int ct = 0; ct < 2; ++ct) wa[ct] = hg_load8(wrow[ct] + kk, kok && cok[ct]);
 #pragma unroll
     for (int ct = 0; ct < 2; ++ct)
 #pragma unroll
       for (int rt = 0; rt < 2; ++rt) {
-        if constexpr (SPLIT) {   // the small pieces first
-          acc[ct][rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wa[ct], xl[rt], acc[ct][rt], 0, 0, 0);
-          acc[ct][rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wa[ct], xm[rt], acc[ct][rt], 0, 0, 0);
-        }
+        // the small pieces first
+        acc[ct][rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wa[ct], xl[rt], acc[ct][rt], 0, 0, 0);
+        acc[ct][rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wa[ct], xm[rt], acc[ct][rt], 0, 0, 0);
         acc[ct][rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wa[ct], xb[rt], acc[ct][rt], 0, 0, 0);
       }
   }
@@ -661,6 +652,48 @@ heads_gemm_wide_kernel(const TX* __restrict__ x, long ldx, long hsx, const bf16_
 
 constexpr int kHWideRows = 96;   // from here on the wide tiles
 
+// For fewer rows: a block owns 16 columns of one head and 16 tokens; its four waves share out K (wave v the steps v, v + 4,
+// ..., four of them in flight) and meet once to add their sums, in the order of the waves.
+template <typename TX, typename TY>
+__global__ void __launch_bounds__(256)
+heads_gemm_few_kernel(const TX* __restrict__ x, long ldx, long hsx, const bf16_t* __restrict__ w, TY* __restrict__ y,
+                      long ldy, long hsy, ProductGate gate, QueryTurn turn, int m, int n, int k, float alpha) {
+  __shared__ float part[4][16][17];
+  const int tid = threadIdx.x, wave = tid / kWave, lane = tid % kWave, r = lane % 16, g = lane / 16;
+  const int h = blockIdx.z, row0 = blockIdx.y * 16, col0 = blockIdx.x * 16;
+  if (col0 >= n) {   // the column of blocks behind the product's
+    turn_queries<TY>(turn, h, row0, m - row0 < 16 ? m - row0 : 16);
+    return;
+  }
+  const TX* xr = x + (size_t)(row0 + r < m ? row0 + r : m - 1) * ldx + (size_t)h * hsx;
+  const bf16_t* wr = w + ((size_t)h * n + (col0 + r < n ? col0 + r : n - 1)) * k;
+  hg_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  for (int k0 = wave * 32; k0 < k; k0 += 512) {
+    HeadPieces<TX> xp[4];
+    HeadPieces<bf16_t> wp[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int at = k0 + i * 128 + 8 * g, kk = at < k ? at : k - 8;   // past the end: the last piece, counted as zeros
+      xp[i].load(xr + kk);
+      wp[i].load(wr + kk);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wp[i].get(true), xp[i].get(k0 + i * 128 + 8 * g < k), acc, 0, 0, 0);
+  }
+  // lane (r, g) holds columns 4g .. 4g + 3 of row r
+#pragma unroll
+  for (int i = 0; i < 4; ++i) part[wave][r][4 * g + i] = acc[i];
+  __syncthreads();
+  const int row = row0 + tid / 16, col = col0 + tid % 16;
+  if (row >= m || col >= n) return;
+  float v = part[0][tid / 16][tid % 16];
+#pragma unroll
+  for (int i = 1; i < 4; ++i) v += part[i][tid / 16][tid % 16];
+  v *= alpha * (gate.g ? gate_value(gate, row, h, col) : 1.f);
+  y[(size_t)row * ldy + (size_t)h * hsy + col] = from_f32<TY>(v);
+}
+
 ATOM_EXPORT int atom_heads_gemm_mfma_supports(int x_dtype, int w_dtype, long x_offset, long ldx, long hsx, int k) {
   if (w_dtype != ATOM_BF16 || k % 8) return 0;
   const long unit = x_dtype == ATOM_BF16 ? 8 : 4;   // elements of 16 bytes
@@ -684,9 +717,6 @@ ATOM_EXPORT int atom_heads_gemm_mfma(const void* x, int x_dtype, long ldx, long 
   if (m == 0) return ATOM_OK;
   dim3 grid((n + 63) / 64 + (rot > 0 ? 1 : 0), (m + 63) / 64, heads), block(256);
   if (grid.y > 65535) return ATOM_TOO_LARGE;
-#define LAUNCH(TX, TY, SPLIT)                                                                                       \
-  hipLaunchKernelGGL((heads_gemm_mfma_kernel<TX, TY, SPLIT>), grid, block, 0, stream, (const TX*)x, ldx, hsx,      \
-                     (const bf16_t*)w, (TY*)y, ldy, hsy, g, q, m, n, k, alpha)
   if (!split && m >= kHWideRows) {
     const long unit = 4;   // entries that are read or written together
     const size_t y_align = (y_dtype == ATOM_BF16 ? 2 : 4) * unit;
@@ -705,17 +735,25 @@ ATOM_EXPORT int atom_heads_gemm_mfma(const void* x, int x_dtype, long ldx, long 
 #undef WIDE
     return launch_status();
   }
-  if (split) {
-    if (y_dtype == ATOM_F32) LAUNCH(float, float, true);
-    else LAUNCH(float, bf16_t, true);
+  if (!split) {
+    grid = dim3((n + 15) / 16 + (rot > 0 ? 1 : 0), (m + 15) / 16, heads);
+#define FEW(TX, TY)                                                                                                 \
+  hipLaunchKernelGGL((heads_gemm_few_kernel<TX, TY>), grid, block, 0, stream, (const TX*)x, ldx, hsx, (const bf16_t*)w, \
+                     (TY*)y, ldy, hsy, g, q, m, n, k, alpha)
+    switch (x_dtype * 2 + y_dtype) {
+      case 0: FEW(float, float); break;
+      case 1: FEW(float, bf16_t); break;
+      case 2: FEW(bf16_t, float); break;
+      default: FEW(bf16_t, bf16_t); break;
+    }
+#undef FEW
     return launch_status();
   }
-  switch (x_dtype * 2 + y_dtype) {
-    case 0: LAUNCH(float, float, false); break;
-    case 1: LAUNCH(float, bf16_t, false); break;
-    case 2: LAUNCH(bf16_t, float, false); break;
-    default: LAUNCH(bf16_t, bf16_t, false); break;
-  }
-#undef LAUNCH
+  if (y_dtype == ATOM_F32)
+    hipLaunchKernelGGL((heads_gemm_split_kernel<float>), grid, block, 0, stream, (const float*)x, ldx, hsx, (const bf16_t*)w,
+                       (float*)y, ldy, hsy, g, q, m, n, k, alpha);
+  else
+    hipLaunchKernelGGL((heads_gemm_split_kernel<bf16_t>), grid, block, 0, stream, (const float*)x, ldx, hsx,
+                       (const bf16_t*)w, (bf16_t*)y, ldy, hsy, g, q, m, n, k, alpha);
   return launch_status();
 }
