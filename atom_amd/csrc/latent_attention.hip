@@ -523,9 +523,11 @@ heads_gemm_split_kernel(const float* __restrict__ x, long ldx, long hsx, const b
   }
 }
 
-// For many rows: a block of 2 x 2 waves owns 128 tokens x 128 columns, a wave 64 x 64 of them, so that a 16-byte piece
-// read feeds four products; the next step's pieces are asked for before this one's products.  `vec`: y, its strides and the
-// gate's suit four columns at a time (n % 4 = 0).
+// For many rows: a block of 2 x 2 waves owns 64 tokens x 128 columns, a wave 32 x 64 of them; K is walked 64 at a time
+// (whole lines of bfloat16 rows), the next 64's pieces asked for before this step's products.  `vec`: y, its strides and the
+// gate's suit eight columns at a time (n % 8 = 0).
+constexpr int kHWideTokens = 64;
+
 template <typename TX>
 struct HeadPieces;
 template <>
@@ -562,90 +564,102 @@ heads_gemm_wide_kernel(const TX* __restrict__ x, long ldx, long hsx, const bf16_
   const int tid = threadIdx.x, wave = tid / kWave, lane = tid % kWave, r = lane % 16, g = lane / 16;
   const int h = blockIdx.z;
   if ((int)blockIdx.x * 128 >= n) {   // the column of blocks behind the product's
-    const int t0 = (int)blockIdx.y * 128;
-    turn_queries<TY>(turn, h, t0, m - t0 < 128 ? m - t0 : 128);
+    const int t0 = (int)blockIdx.y * kHWideTokens;
+    turn_queries<TY>(turn, h, t0, m - t0 < kHWideTokens ? m - t0 : kHWideTokens);
     return;
   }
-  const int row0 = blockIdx.y * 128 + (wave / 2) * 64;
+  constexpr int RT = kHWideTokens / 32, CT = 4;   // 16-row and 16-column tiles of a wave
+  const int row0 = blockIdx.y * kHWideTokens + (wave / 2) * (RT * 16);
   const int col0 = blockIdx.x * 128 + (wave % 2) * 64;
   // rows and columns beyond the product's are read as its last ones and not written
-  const TX* xrow[4];
-  const bf16_t* wrow[4];
+  const TX* xrow[RT];
+  const bf16_t* wrow[CT];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int row = row0 + i * 16 + r < m ? row0 + i * 16 + r : m - 1;
-    const int col = col0 + i * 16 + r < n ? col0 + i * 16 + r : n - 1;
-    xrow[i] = x + (size_t)row * ldx + (size_t)h * hsx;
-    wrow[i] = w + ((size_t)h * n + col) * k;
-  }
-  hg_f32x4 acc[4][4];   // [16 columns][16 rows]
+  for (int j = 0; j < RT; ++j)
+    xrow[j] = x + (size_t)(row0 + j * 16 + r < m ? row0 + j * 16 + r : m - 1) * ldx + (size_t)h * hsx;
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
+  for (int i = 0; i < CT; ++i)
+    wrow[i] = w + ((size_t)h * n + (col0 + i * 16 + r < n ? col0 + i * 16 + r : n - 1)) * k;
+  hg_f32x4 acc[CT][RT];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) acc[i][j] = hg_f32x4{0.f, 0.f, 0.f, 0.f};
-  HeadPieces<TX> xp[2][4];
-  HeadPieces<bf16_t> wp[2][4];
+  for (int i = 0; i < CT; ++i)
+#pragma unroll
+    for (int j = 0; j < RT; ++j) acc[i][j] = hg_f32x4{0.f, 0.f, 0.f, 0.f};
+  HeadPieces<TX> xp[2][2][RT];
+  HeadPieces<bf16_t> wp[2][2][CT];
   auto fetch = [&](int buffer, int k0) {
-    const int kk = k0 + 8 * g < k ? k0 + 8 * g : k - 8;   // past the end: the last piece, which counts as zeros
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      xp[buffer][i].load(xrow[i] + kk);
-      wp[buffer][i].load(wrow[i] + kk);
+    for (int s = 0; s < 2; ++s) {
+      const int at = k0 + s * 32 + 8 * g, kk = at < k ? at : k - 8;   // past the end: the last piece, counted as zeros
+#pragma unroll
+      for (int j = 0; j < RT; ++j) xp[buffer][s][j].load(xrow[j] + kk);
+#pragma unroll
+      for (int i = 0; i < CT; ++i) wp[buffer][s][i].load(wrow[i] + kk);
     }
   };
   auto multiply = [&](int buffer, int k0) {
-    const bool ok = k0 + 8 * g < k;
-    hg_bf16x8 xb[4];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) xb[j] = xp[buffer][j].get(ok);
+    for (int s = 0; s < 2; ++s) {
+      const bool ok = k0 + s * 32 + 8 * g < k;
+      hg_bf16x8 xb[RT];
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
+      for (int j = 0; j < RT; ++j) xb[j] = xp[buffer][s][j].get(ok);
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wp[buffer][i].get(true), xb[j], acc[i][j], 0, 0, 0);
+      for (int i = 0; i < CT; ++i)
+#pragma unroll
+        for (int j = 0; j < RT; ++j)
+          acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wp[buffer][s][i].get(true), xb[j], acc[i][j], 0, 0, 0);
+    }
   };
   fetch(0, 0);
-  for (int k0 = 0; k0 < k; k0 += 64) {
-    fetch(1, k0 + 32);
+  for (int k0 = 0; k0 < k; k0 += 128) {
+    fetch(1, k0 + 64);
+    __builtin_amdgcn_sched_barrier(0);
     multiply(0, k0);
-    fetch(0, k0 + 64);
-    multiply(1, k0 + 32);
+    fetch(0, k0 + 128);
+    __builtin_amdgcn_sched_barrier(0);
+    multiply(1, k0 + 64);
   }
-  // lane (r, g) holds columns col0 + 16 i + 4g .. + 3 of row row0 + 16 j + r
+  // lane (r, g) holds columns col0 + 16 i + 4g .. + 3 of row row0 + 16 j + r; through LDS, so that whole lines are written
+  __shared__ __attribute__((aligned(16))) float tile[kHWideTokens][128 + 4];
 #pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int row = row0 + j * 16 + r;
-    if (row >= m) continue;
+  for (int j = 0; j < RT; ++j)
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int col = col0 + i * 16 + 4 * g;
-      if (col >= n) continue;
-      TY* dst = y + (size_t)row * ldy + (size_t)h * hsy + col;
-      hg_f32x4 v = acc[i][j] * alpha;
-      if (vec) {
-        if (gate.g) {
-          if (gate.csg) {
-            const hg_f32x4 gv = *reinterpret_cast<const hg_f32x4*>(gate.g + row * gate.ldg + (size_t)h * gate.hsg + col);
+    for (int i = 0; i < CT; ++i)
+      *reinterpret_cast<hg_f32x4*>(&tile[(wave / 2) * (RT * 16) + j * 16 + r][(wave % 2) * 64 + i * 16 + 4 * g]) = acc[i][j] * alpha;
+  __syncthreads();
+  const int c = (tid % 16) * 8, col = blockIdx.x * 128 + c;
+  for (int t = tid / 16; t < kHWideTokens; t += 16) {
+    const int row = (int)blockIdx.y * kHWideTokens + t;
+    if (row >= m || col >= n) break;
+    float v[8];
 #pragma unroll
-            for (int q = 0; q < 4; ++q) v[q] *= 1.f / (1.f + expf(-gv[q]));
-          } else {
-            v *= gate_value(gate, row, h, 0);
-          }
-        }
-        if constexpr (sizeof(TY) == 2) {
-          typedef __attribute__((ext_vector_type(4))) __bf16 hg_bf16x4;
-          hg_bf16x4 o;
+    for (int q = 0; q < 8; ++q) v[q] = tile[t][c + q];
+    TY* dst = y + (size_t)row * ldy + (size_t)h * hsy + col;
+    if (vec) {
+      if (gate.g && gate.csg) {
+        const float* gp = gate.g + row * gate.ldg + (size_t)h * gate.hsg + col;
+        const hg_f32x4 ga = *reinterpret_cast<const hg_f32x4*>(gp), gb = *reinterpret_cast<const hg_f32x4*>(gp + 4);
 #pragma unroll
-          for (int q = 0; q < 4; ++q) o[q] = static_cast<__bf16>(v[q]);
-          *reinterpret_cast<hg_bf16x4*>(dst) = o;
-        } else {
-          *reinterpret_cast<hg_f32x4*>(dst) = v;
-        }
-      } else {
+        for (int q = 0; q < 8; ++q) v[q] *= 1.f / (1.f + expf(-(q < 4 ? ga[q] : gb[q - 4])));
+      } else if (gate.g) {
+        const float f = gate_value(gate, row, h, 0);
 #pragma unroll
-        for (int q = 0; q < 4; ++q)
-          if (col + q < n) dst[q] = from_f32<TY>(v[q] * (gate.g ? gate_value(gate, row, h, col + q) : 1.f));
+        for (int q = 0; q < 8; ++q) v[q] *= f;
       }
+      if constexpr (sizeof(TY) == 2) {
+        hg_bf16x8 o;
+#pragma unroll
+        for (int q = 0; q < 8; ++q) o[q] = static_cast<__bf16>(v[q]);
+        *reinterpret_cast<hg_bf16x8*>(dst) = o;
+      } else {
+        *reinterpret_cast<hg_f32x4*>(dst) = hg_f32x4{v[0], v[1], v[2], v[3]};
+        *reinterpret_cast<hg_f32x4*>(dst + 4) = hg_f32x4{v[4], v[5], v[6], v[7]};
+      }
+    } else {
+#pragma unroll
+      for (int q = 0; q < 8; ++q)
+        if (col + q < n) dst[q] = from_f32<TY>(v[q] * (gate.g ? gate_value(gate, row, h, col + q) : 1.f));
     }
   }
 }
@@ -718,11 +732,10 @@ ATOM_EXPORT int atom_heads_gemm_mfma(const void* x, int x_dtype, long ldx, long 
   dim3 grid((n + 63) / 64 + (rot > 0 ? 1 : 0), (m + 63) / 64, heads), block(256);
   if (grid.y > 65535) return ATOM_TOO_LARGE;
   if (!split && m >= kHWideRows) {
-    const long unit = 4;   // entries that are read or written together
-    const size_t y_align = (y_dtype == ATOM_BF16 ? 2 : 4) * unit;
-    const int vec = n % unit == 0 && ldy % unit == 0 && hsy % unit == 0 && (size_t)y % y_align == 0 &&
-                    (g.g == nullptr || g.csg == 0 || ((size_t)g.g % 16 == 0 && g.ldg % unit == 0 && g.hsg % unit == 0));
-    grid = dim3((n + 127) / 128 + (rot > 0 ? 1 : 0), (m + 127) / 128, heads);
+    const long unit = 8;   // entries that are read or written together
+    const int vec = n % unit == 0 && ldy % unit == 0 && hsy % unit == 0 && (size_t)y % 16 == 0 &&
+                    (g.g == nullptr || g.csg == 0 || ((size_t)g.g % 16 == 0 && g.ldg % 4 == 0 && g.hsg % 4 == 0));
+    grid = dim3((n + 127) / 128 + (rot > 0 ? 1 : 0), (m + kHWideTokens - 1) / kHWideTokens, heads);
 #define WIDE(TX, TY)                                                                                                \
   hipLaunchKernelGGL((heads_gemm_wide_kernel<TX, TY>), grid, block, 0, stream, (const TX*)x, ldx, hsx, (const bf16_t*)w, \
                      (TY*)y, ldy, hsy, g, q, m, n, k, alpha, vec)
