@@ -171,6 +171,7 @@ class StateSlots:
 @dataclass
 class _Request:
     tables: list[list[int]]   # per group: page id per page index, -1 where none is held
+    given: list[int]          # per group: places of the table before this one hold no page any more; all from it on do
     slot: int
     fresh: bool = True        # no step has run for it yet
     serial: int = 0           # unique per ``open``: a request id that is opened again gets a new one
@@ -218,7 +219,7 @@ class CacheManager:
             raise KeyError(f"request {req_id!r} is already open")
         slot = self.slots.claim()
         self._opened += 1
-        self._requests[req_id] = _Request([[] for _ in self.groups], slot, serial=self._opened)
+        self._requests[req_id] = _Request([[] for _ in self.groups], [0] * len(self.groups), slot, serial=self._opened)
         return slot
 
     def close(self, req_id) -> None:
@@ -275,12 +276,8 @@ class CacheManager:
                 # nothing is given back before the request ends: the table has no gaps
                 out.append(max(0, last + 1 - len(table)))
                 continue
-            first = self._first_page_needed(gi, cached)
-            need = 0
-            for idx in range(first, last + 1):
-                if idx >= len(table) or table[idx] < 0:
-                    need += 1
-            out.append(need)
+            # a window group's table holds every page from the first one still needed to its end
+            out.append(max(0, last + 1 - max(len(table), self._first_page_needed(gi, cached))))
         return out
 
     def can_cover(self, req_id, cached: int, upto: int, reserve: int | None = None) -> bool:
@@ -304,15 +301,15 @@ class CacheManager:
                     table.append(self.pools[gi].take())
                 continue
             first = self._first_page_needed(gi, cached)
-            while len(table) <= last:
+            if first < req.given[gi]:
+                # a page wholly behind the cached tokens can only be missing because the window passed it; a query
+                # that needs it again would read nothing
+                raise AssertionError(f"request {req_id!r}: page {first} was given back and is needed again")
+            while len(table) < first:        # places that no query sees any more: never filled
                 table.append(-1)
-            for idx in range(first, last + 1):
-                if table[idx] < 0:
-                    if idx * g.page_size + g.page_size <= cached:
-                        # a page wholly behind the cached tokens can only be missing because the
-                        # window passed it; a query that needs it again would read nothing
-                        raise AssertionError(f"request {req_id!r}: page {idx} was given back and is needed again")
-                    table[idx] = self.pools[gi].take()
+                req.given[gi] = len(table)
+            while len(table) <= last:
+                table.append(self.pools[gi].take())
 
     # ------------------------------------------------------------------ prefix cache
 
@@ -387,12 +384,12 @@ class CacheManager:
         for gi, g in enumerate(self.groups):
             if g.keeps_all:
                 continue
-            first = self._first_page_needed(gi, cached_after)
             table = req.tables[gi]
-            for idx in range(min(first, len(table))):
-                if table[idx] >= 0:
-                    self.pools[gi].give(table[idx])
-                    table[idx] = -1
+            upto = min(self._first_page_needed(gi, cached_after), len(table))
+            for idx in range(req.given[gi], upto):
+                self.pools[gi].give(table[idx])
+                table[idx] = -1
+            req.given[gi] = max(req.given[gi], upto)
 
     def awaited_position(self, req_id) -> int | None:
         """The position whose token ``commit`` took as not yet known, if there is one."""
@@ -416,6 +413,11 @@ class CacheManager:
     def slot_mapping(self, req_id, group: int, start: int, count: int) -> np.ndarray:
         """Cache slot (page * page_size + offset) of positions start .. start + count - 1."""
         g = self.groups[group]
+        if count == 1:
+            page = self._requests[req_id].tables[group][start // g.page_size]
+            if page < 0:
+                raise AssertionError(f"request {req_id!r}: position {start} has no page")
+            return np.asarray([page * g.page_size + start % g.page_size], dtype=np.int32)
         table = np.asarray(self._requests[req_id].tables[group], dtype=np.int64)
         pos = np.arange(start, start + count, dtype=np.int64)
         pages = table[pos // g.page_size]

@@ -211,12 +211,13 @@ class DecodeGraphs:
                 slot_arrays[gi][first:first + k] = mgr.slot_mapping(e.req_id, gi, c, k)
                 bt, state = tables[gi], cap.row_state[gi]
                 held, serial = state[row], mgr.serial(e.req_id)
-                windowed = not mgr.groups[gi].keeps_all
                 if table[(c + k - 1) // page_size] < 0:
                     raise AssertionError(f"request {e.req_id!r}: position {c + k - 1} has no page")
-                if not windowed and held is not None and held[0] == serial and held[1] <= len(table):
-                    if held[1] < len(table):     # pages appended since the row was last written
-                        bt[row, held[1]:len(table)] = table[held[1]:]
+                if held is not None and held[0] == serial and held[1] <= len(table):
+                    # pages appended since the row was last written; places whose pages a window has passed meanwhile
+                    # keep their old numbers, which no query's keys name any more
+                    if held[1] < len(table):
+                        bt[row, held[1]:len(table)] = [max(page, 0) for page in table[held[1]:]]
                 else:
                     line = np.asarray(table, dtype=np.int32)
                     bt[row, :len(table)] = np.where(line < 0, 0, line)
