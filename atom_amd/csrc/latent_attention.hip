@@ -13,6 +13,8 @@
 //                       absorbing product takes the rotation of the queries' rotated parts with it (QueryTurn)
 //   latent_attention    scores, softmax with sink, weighted sum; any sizes, float32 or bfloat16 pages
 //
+//   rotation_table      the cosines and sines of a step's tokens, which every layer with the same rotation reads
+//
 // Rotation: entries (2i, 2i + 1) of the rotated part are a pair; its angle is position * freq[i], formed in
 // float64 from a float64 table and reduced to (-pi, pi] before the float32 sine and cosine; both are multiplied
 // by `mult`.
@@ -28,14 +30,35 @@ __device__ __forceinline__ void pair_angle(int position, double freq, float mult
   *s = sf * mult;
 }
 
+// table[t][i] = (cos, sin) of token t's angle of pair i
+__global__ void __launch_bounds__(256)
+rotation_table_kernel(const int* __restrict__ positions, const double* __restrict__ freq, float mult, float2* __restrict__ table,
+                      int tokens, int pairs) {
+  const long at = (long)blockIdx.x * 256 + threadIdx.x;
+  if (at >= (long)tokens * pairs) return;
+  float c, s;
+  pair_angle(positions[at / pairs], freq[at % pairs], mult, &c, &s);
+  table[at] = make_float2(c, s);
+}
+
+ATOM_EXPORT int atom_rotation_table(const int* positions, const double* freq, float mult, void* table, int tokens, int pairs,
+                                    hipStream_t stream) {
+  if (tokens < 0 || pairs <= 0 || positions == nullptr || freq == nullptr || table == nullptr) return ATOM_BAD_SHAPE;
+  if (tokens == 0) return ATOM_OK;
+  const long blocks = ((long)tokens * pairs + 255) / 256;
+  if (blocks > 0x7fffffffL / 256) return ATOM_TOO_LARGE;
+  hipLaunchKernelGGL(rotation_table_kernel, dim3((unsigned)blocks), dim3(256), 0, stream, positions, freq, mult,
+                     (float2*)table, tokens, pairs);
+  return launch_status();
+}
+
 // proj [tokens, ld] float32 holds, where asked for, the latent of the queries at cq_off (cq_rank entries) and the
 // down-projection of the keys at kv_off (rank entries, then rot).  A block a token.
 template <typename T>
 __global__ void __launch_bounds__(256)
 latent_prepare_kernel(const float* __restrict__ proj, int ld, int cq_off, int cq_rank, const float* __restrict__ cq_w,
                       T* __restrict__ cq, int kv_off, int rank, int rot, int rot_dims, const float* __restrict__ norm_w,
-                      float eps, const double* __restrict__ freq, float mult, const int* __restrict__ positions,
-                      const int* __restrict__ slots, T* __restrict__ pages) {
+                      float eps, const float2* __restrict__ turns, const int* __restrict__ slots, T* __restrict__ pages) {
   __shared__ float scratch[2][4];
   const int t = blockIdx.x;
   const int tid = threadIdx.x;
@@ -53,10 +76,9 @@ latent_prepare_kernel(const float* __restrict__ proj, int ld, int cq_off, int cq
     for (int i = 255 - tid; i < rot; i += 256) {
       float v = row[kv_off + rank + i];
       if (i < rot_dims) {
-        float c, s;
-        pair_angle(positions[t], freq[i >> 1], mult, &c, &s);
+        const float2 cs = turns[(size_t)t * (rot_dims / 2) + (i >> 1)];
         const float other = row[kv_off + rank + (i ^ 1)];
-        v = (i & 1) ? v * c + other * s : v * c - other * s;
+        v = (i & 1) ? v * cs.x + other * cs.y : v * cs.x - other * cs.y;
       }
       dst[i] = from_f32<T>(v);
     }
@@ -84,20 +106,20 @@ latent_prepare_kernel(const float* __restrict__ proj, int ld, int cq_off, int cq
 
 ATOM_EXPORT int atom_latent_prepare(const float* proj, int ld, int cq_off, int cq_rank, const float* cq_w, void* cq,
                                     int kv_off, int rank, int rot, int rot_dims, const float* norm_w, float eps,
-                                    const double* freq, float mult, const int* positions, const int* slots, void* pages,
-                                    int dtype, int tokens, hipStream_t stream) {
+                                    const void* turns, const int* slots, void* pages, int dtype, int tokens,
+                                    hipStream_t stream) {
   if (tokens < 0 || ld <= 0 || cq_rank < 0 || proj == nullptr) return ATOM_BAD_SHAPE;
   if (cq_rank > 0 && (cq_off < 0 || cq_off + cq_rank > ld || cq_w == nullptr || cq == nullptr)) return ATOM_BAD_SHAPE;
   if (slots != nullptr) {
     if (rot < 0 || rank <= 0 || rot_dims < 0 || rot_dims > rot || (rot_dims & 1)) return ATOM_BAD_SHAPE;
     if (kv_off < 0 || kv_off + rank + rot > ld) return ATOM_BAD_SHAPE;
-    if (norm_w == nullptr || positions == nullptr || pages == nullptr) return ATOM_BAD_SHAPE;
-    if (rot_dims > 0 && freq == nullptr) return ATOM_BAD_SHAPE;
+    if (norm_w == nullptr || pages == nullptr) return ATOM_BAD_SHAPE;
+    if (rot_dims > 0 && turns == nullptr) return ATOM_BAD_SHAPE;
   }
   if (tokens == 0 || (cq_rank == 0 && slots == nullptr)) return ATOM_OK;
   ATOM_DISPATCH_DTYPE(dtype, hipLaunchKernelGGL((latent_prepare_kernel<T>), dim3(tokens), dim3(256), 0, stream, proj, ld,
                                                  cq_off, cq_rank, cq_w, (T*)cq, kv_off, rank, rot, rot_dims, norm_w, eps,
-                                                 freq, mult, positions, slots, (T*)pages));
+                                                 (const float2*)turns, slots, (T*)pages));
   return launch_status();
 }
 
@@ -107,10 +129,9 @@ struct QueryTurn {
   const float* x;        // [tokens, ..] float32: head h's rotated part at t * ldx + h * hsx
   void* out;             // the product's output type: at t * ldo + h * hso
   long ldx, hsx, ldo, hso;
-  const double* freq;
-  const int* positions;
+  const float2* turns;   // [tokens, rot_dims / 2]: rotation_table
   int rot, rot_dims;     // rot 0: nothing to do
-  float mult, scale;
+  float scale;
 };
 
 // Tokens t0 .. t0 + count - 1 of head h, by a block of 256 threads: an item is a pair of neighbours (or a last single).
@@ -124,10 +145,9 @@ __device__ __forceinline__ void turn_queries(const QueryTurn& q, int h, int t0, 
     const bool both = i + 1 < q.rot;
     float u = src[0], v = both ? src[1] : 0.f;
     if (i < q.rot_dims) {
-      float c, s;
-      pair_angle(q.positions[t], q.freq[i >> 1], q.mult, &c, &s);
-      const float a = u * c - v * s;
-      v = v * c + u * s;
+      const float2 cs = q.turns[(size_t)t * (q.rot_dims / 2) + (i >> 1)];
+      const float a = u * cs.x - v * cs.y;
+      v = v * cs.x + u * cs.y;
       u = a;
     }
     dst[0] = from_f32<T>(u * q.scale);
@@ -252,29 +272,28 @@ heads_rows_kernel(const TX* __restrict__ x, long ldx, long hsx, const TW* __rest
 
 // The options of a per-head product from the host's plain arguments; false where they do not fit together.
 static bool product_options(const float* gate, long ldg, int hsg, int csg, const float* qx, long ldqx, long hsqx, void* qout,
-                            long ldqo, long hsqo, int rot, int rot_dims, const double* freq, float mult, float scale,
-                            const int* positions, ProductGate* g, QueryTurn* q) {
+                            long ldqo, long hsqo, int rot, int rot_dims, const void* turns, float scale, ProductGate* g,
+                            QueryTurn* q) {
   if (gate != nullptr && (ldg < 0 || hsg < 0 || csg < 0)) return false;
   *g = ProductGate{gate, ldg, hsg, csg};
   if (rot < 0 || rot_dims < 0 || rot_dims > rot || (rot_dims & 1)) return false;
-  if (rot > 0 && (qx == nullptr || qout == nullptr || positions == nullptr)) return false;
-  if (rot_dims > 0 && freq == nullptr) return false;
-  *q = QueryTurn{qx, qout, ldqx, hsqx, ldqo, hsqo, freq, positions, rot, rot_dims, mult, scale};
+  if (rot > 0 && (qx == nullptr || qout == nullptr)) return false;
+  if (rot_dims > 0 && turns == nullptr) return false;
+  *q = QueryTurn{qx, qout, ldqx, hsqx, ldqo, hsqo, (const float2*)turns, rot, rot_dims, scale};
   return true;
 }
 
 ATOM_EXPORT int atom_heads_gemm(const void* x, int x_dtype, long ldx, long hsx, const void* w, int w_dtype, void* y,
                                 int y_dtype, long ldy, long hsy, const float* gate, long ldg, int hsg, int csg,
                                 const float* qx, long ldqx, long hsqx, void* qout, long ldqo, long hsqo, int rot,
-                                int rot_dims, const double* freq, float mult, float scale, const int* positions, int heads,
-                                int m, int n, int k, float alpha, hipStream_t stream) {
+                                int rot_dims, const void* turns, float scale, int heads, int m, int n, int k, float alpha,
+                                hipStream_t stream) {
   if (m < 0 || n <= 0 || k <= 0 || heads <= 0 || heads > 65535) return ATOM_BAD_SHAPE;
   if (x == nullptr || w == nullptr || y == nullptr) return ATOM_BAD_SHAPE;
   if ((unsigned)x_dtype > 1u || (unsigned)w_dtype > 1u || (unsigned)y_dtype > 1u) return ATOM_BAD_DTYPE;
   ProductGate g;
   QueryTurn q;
-  if (!product_options(gate, ldg, hsg, csg, qx, ldqx, hsqx, qout, ldqo, hsqo, rot, rot_dims, freq, mult, scale, positions,
-                       &g, &q))
+  if (!product_options(gate, ldg, hsg, csg, qx, ldqx, hsqx, qout, ldqo, hsqo, rot, rot_dims, turns, scale, &g, &q))
     return ATOM_BAD_SHAPE;
   if (m == 0) return ATOM_OK;
   const bool few = m <= kHFewRows;
@@ -612,13 +631,19 @@ heads_gemm_wide_kernel(const TX* __restrict__ x, long ldx, long hsx, const bf16_
     }
   };
   fetch(0, 0);
-  for (int k0 = 0; k0 < k; k0 += 128) {
-    fetch(1, k0 + 64);
-    __builtin_amdgcn_sched_barrier(0);
-    multiply(0, k0);
-    fetch(0, k0 + 128);
-    __builtin_amdgcn_sched_barrier(0);
-    multiply(1, k0 + 64);
+  if (k <= 128) {   // nothing behind the second fetch: no third one that would only be thrown away
+    fetch(1, 64);
+    multiply(0, 0);
+    multiply(1, 64);
+  } else {
+    for (int k0 = 0; k0 < k; k0 += 128) {
+      fetch(1, k0 + 64);
+      __builtin_amdgcn_sched_barrier(0);
+      multiply(0, k0);
+      fetch(0, k0 + 128);
+      __builtin_amdgcn_sched_barrier(0);
+      multiply(1, k0 + 64);
+    }
   }
   // lane (r, g) holds columns col0 + 16 i + 4g .. + 3 of row row0 + 16 j + r; through LDS, so that whole lines are written
   __shared__ __attribute__((aligned(16))) float tile[kHWideTokens][128 + 4];
@@ -717,16 +742,15 @@ ATOM_EXPORT int atom_heads_gemm_mfma_supports(int x_dtype, int w_dtype, long x_o
 ATOM_EXPORT int atom_heads_gemm_mfma(const void* x, int x_dtype, long ldx, long hsx, const void* w, void* y, int y_dtype,
                                      long ldy, long hsy, const float* gate, long ldg, int hsg, int csg, const float* qx,
                                      long ldqx, long hsqx, void* qout, long ldqo, long hsqo, int rot, int rot_dims,
-                                     const double* freq, float mult, float scale, const int* positions, int heads, int m,
-                                     int n, int k, float alpha, int split, hipStream_t stream) {
+                                     const void* turns, float scale, int heads, int m, int n, int k, float alpha, int split,
+                                     hipStream_t stream) {
   if (m < 0 || n <= 0 || k <= 0 || heads <= 0 || heads > 65535 || (k % 8)) return ATOM_BAD_SHAPE;
   if (split && x_dtype != ATOM_F32) return ATOM_UNSUPPORTED;   // only a float32 input has pieces to split into
   if (x == nullptr || w == nullptr || y == nullptr) return ATOM_BAD_SHAPE;
   if ((unsigned)x_dtype > 1u || (unsigned)y_dtype > 1u) return ATOM_BAD_DTYPE;
   ProductGate g;
   QueryTurn q;
-  if (!product_options(gate, ldg, hsg, csg, qx, ldqx, hsqx, qout, ldqo, hsqo, rot, rot_dims, freq, mult, scale, positions,
-                       &g, &q))
+  if (!product_options(gate, ldg, hsg, csg, qx, ldqx, hsqx, qout, ldqo, hsqo, rot, rot_dims, turns, scale, &g, &q))
     return ATOM_BAD_SHAPE;
   if (m == 0) return ATOM_OK;
   dim3 grid((n + 63) / 64 + (rot > 0 ? 1 : 0), (m + 63) / 64, heads), block(256);

@@ -99,18 +99,15 @@ class AttentionMeta:
 @dataclass
 class QueryTurn:
     """The rotated parts of queries, which a per-head product (``HipKernels.heads_gemm``) turns and writes beside its
-    output: head h's ``rot`` entries of token t at ``x_offset + t * ldx + h * hsx`` of its float32 input, the first
-    ``rot_dims`` of them rotated in neighbouring pairs by ``positions[t] * freq``, times ``scale``, go to ``y_offset + t
+    output: head h's ``rot`` entries of token t at ``x_offset + t * ldx + h * hsx`` of its float32 input, the first of them
+    rotated in neighbouring pairs as ``turns`` says (``HipKernels.rotation_table``; None: none), times ``scale``, go to ``y_offset + t
     * ldy + h * hsy`` of its output."""
 
     x_offset: int
     y_offset: int
     rot: int
-    rot_dims: int
-    freq: torch.Tensor | None
-    mult: float
+    turns: torch.Tensor | None
     scale: float
-    positions: torch.Tensor
 
 
 class DeferredSum:
@@ -205,7 +202,7 @@ class HipKernels:
                    "atom_attention_prefill_tile_rows", "atom_attention_decode_fused",
                    "atom_attention_decode_fused_supports", "atom_gemm_rows", "atom_gemm_rows_parts",
                    "atom_gemm_rows_supports", "atom_gemm_tile", "atom_gemm_tile_splits", "atom_gemm_tile_supports",
-                   "atom_layernorm", "atom_embedding_scaled", "atom_sum_concat", "atom_gated_act", "atom_latent_prepare",
+                   "atom_layernorm", "atom_embedding_scaled", "atom_sum_concat", "atom_gated_act", "atom_latent_prepare", "atom_rotation_table",
                    "atom_heads_gemm", "atom_latent_attention", "atom_conv_silu_state", "atom_delta_rule",
                    "atom_delta_out", "atom_router_choose", "atom_experts_gate_up", "atom_experts_down",
                    "atom_latent_attention_tile", "atom_latent_tile_supports", "atom_latent_merge",
@@ -1038,12 +1035,23 @@ class HipKernels:
 
     # ------------------------------------------------------------------ attention over a cache of latents
 
-    def latent_prepare(self, proj, pages, slots, positions, kv_off: int, rank: int, rot: int, norm_weight, eps: float,
-                       freq=None, rot_dims: int = 0, mult: float = 1.0, query=None):
+    def rotation_table(self, positions, freq, mult: float = 1.0):
+        """float32 [tokens, pairs, 2]: the cosine and sine of ``positions[t] * freq[i]``, times ``mult``."""
+        tokens, pairs = positions.numel(), freq.numel()
+        self._check("positions", positions, torch.int32, (tokens,))
+        self._check("rotation frequencies", freq, torch.float64, (pairs,))
+        table = torch.empty((tokens, pairs, 2), dtype=torch.float32, device=positions.device)
+        self._done("rotation_table", self.lib.atom_rotation_table(_ptr(positions), _ptr(freq), ctypes.c_float(mult),
+                                                                  _ptr(table), tokens, pairs, self._stream()))
+        return table
+
+    def latent_prepare(self, proj, pages, slots, kv_off: int, rank: int, rot: int, norm_weight, eps: float, turns=None,
+                       query=None):
         """From the float32 product ``proj`` [tokens, *]: the RMS-normed latent (``rank`` entries at ``kv_off``) and the
-        rotated shared key part (the ``rot`` entries after it) go to row ``slots[t]`` of ``pages`` (``slots`` None: no
-        keys are projected here).  ``query`` = (offset, weight, out): the latent that queries are projected up from,
-        RMS-normed with ``weight`` into ``out`` [tokens, its size].  ``eps`` is both norms'."""
+        shared key part (the ``rot`` entries after it, rotated as ``turns`` says, a ``rotation_table``) go to row
+        ``slots[t]`` of ``pages`` (``slots`` None: no keys are projected here).  ``query`` = (offset, weight, out): the
+        latent that queries are projected up from, RMS-normed with ``weight`` into ``out`` [tokens, its size].  ``eps`` is
+        both norms'."""
         tokens, ld = proj.shape
         self._check("projections", proj, torch.float32)
         cq_off, cq_rank, cq_weight, cq = 0, 0, None, None
@@ -1054,23 +1062,31 @@ class HipKernels:
             self._check("query latent", cq, (torch.float32, torch.bfloat16), (tokens, cq_rank))
             if cq_off < 0 or cq_off + cq_rank > ld:
                 raise KernelError("latent_prepare: the query latent's columns are not in the product")
+        pairs = 0
         if slots is not None:
             self._check("latent norm weight", norm_weight, torch.float32, (rank,))
-            self._check("positions", positions, torch.int32, (tokens,))
             self._check("slot mapping", slots, torch.int32, (tokens,))
             self._check("latent pages", pages, cq.dtype if cq is not None else (torch.float32, torch.bfloat16),
                         (None, None, rank + rot))
             if kv_off < 0 or kv_off + rank + rot > ld:
                 raise KernelError("latent_prepare: the keys' columns are not in the product")
-            if rot_dims:
-                self._check("rotation frequencies", freq, torch.float64, (rot_dims // 2,))
+            pairs = self._pairs(turns, tokens, rot)
         elif query is None:
             return
         self._done("latent_prepare", self.lib.atom_latent_prepare(
-            _ptr(proj), ld, cq_off, cq_rank, _ptr(cq_weight), _ptr(cq), kv_off, rank, rot, rot_dims,
-            _ptr(norm_weight) if slots is not None else None, ctypes.c_float(eps), _ptr(freq) if rot_dims else None,
-            ctypes.c_float(mult), _ptr(positions), _ptr(slots), _ptr(pages) if slots is not None else None,
-            self._code(cq if cq is not None else pages), tokens, self._stream()))
+            _ptr(proj), ld, cq_off, cq_rank, _ptr(cq_weight), _ptr(cq), kv_off, rank, rot, 2 * pairs,
+            _ptr(norm_weight) if slots is not None else None, ctypes.c_float(eps), _ptr(turns) if pairs else None,
+            _ptr(slots), _ptr(pages) if slots is not None else None, self._code(cq if cq is not None else pages), tokens,
+            self._stream()))
+
+    def _pairs(self, turns, tokens: int, rot: int) -> int:
+        """How many pairs of a rotated part of ``rot`` entries a rotation table turns."""
+        if turns is None:
+            return 0
+        self._check("rotation table", turns, torch.float32, (tokens, None, 2))
+        if 2 * turns.shape[1] > rot:
+            raise KernelError(f"{turns.shape[1]} pairs do not fit a rotated part of {rot} entries")
+        return turns.shape[1]
 
     def heads_gemm(self, x, x_offset: int, ldx: int, hsx: int, weight, y, y_offset: int, ldy: int, hsy: int, heads: int,
                    m: int, n: int, k: int, alpha: float = 1.0, gate=None, gate_offset: int = 0, ldg: int = 0,
@@ -1100,20 +1116,17 @@ class HipKernels:
         options = [gp, ctypes.c_long(ldg), n if gate_entries else 1, 1 if gate_entries else 0]
         if turn is not None and turn.rot:
             self._check("queries to turn", x, torch.float32)
-            self._check("positions", turn.positions, torch.int32, (m,))
-            if turn.rot_dims:
-                self._check("rotation frequencies", turn.freq, torch.float64, (turn.rot_dims // 2,))
+            pairs = self._pairs(turn.turns, m, turn.rot)
             if m and (turn.x_offset + (m - 1) * ldx + (heads - 1) * hsx + turn.rot > x.numel()
                       or turn.y_offset + (m - 1) * ldy + (heads - 1) * hsy + turn.rot > y.numel()):
                 raise KernelError("heads_gemm: the queries to turn do not lie in the product's tensors")
             options += [ctypes.c_void_p(x.data_ptr() + x.element_size() * turn.x_offset), ctypes.c_long(ldx),
                         ctypes.c_long(hsx), ctypes.c_void_p(y.data_ptr() + y.element_size() * turn.y_offset),
-                        ctypes.c_long(ldy), ctypes.c_long(hsy), turn.rot, turn.rot_dims,
-                        _ptr(turn.freq) if turn.rot_dims else None, ctypes.c_float(turn.mult), ctypes.c_float(turn.scale),
-                        _ptr(turn.positions)]
+                        ctypes.c_long(ldy), ctypes.c_long(hsy), turn.rot, 2 * pairs, _ptr(turn.turns) if pairs else None,
+                        ctypes.c_float(turn.scale)]
         else:
             zero = ctypes.c_long(0)
-            options += [None, zero, zero, None, zero, zero, 0, 0, None, ctypes.c_float(1.0), ctypes.c_float(1.0), None]
+            options += [None, zero, zero, None, zero, zero, 0, 0, None, ctypes.c_float(1.0)]
         xp = ctypes.c_void_p(x.data_ptr() + x.element_size() * x_offset)
         yp = ctypes.c_void_p(y.data_ptr() + y.element_size() * y_offset)
         split = bool(exact and x.dtype == torch.float32)

@@ -114,14 +114,23 @@ class LatentAttention(Mixer):
             ctx.memo[key] = meta
         return meta
 
+    def _turns(self, ctx):
+        """The step's cosines and sines, formed by the first layer with this rotation and read by the others."""
+        rope = self.rope
+        if rope is None or not rope.dims:
+            return None
+        key = ("rotation table", rope.identity)
+        if key not in ctx.memo:
+            ctx.memo[key] = ctx.ops.rotation_table(ctx.positions, rope.freq, rope.mult)
+        return ctx.memo[key]
+
     def forward(self, ctx, x, cache):
         ops = ctx.ops
         T = x.shape[0]
         H, d, r, dv, rank = self.num_heads, self.head_dim, self.rot_dim, self.value_dim, self.kv_rank
         width = rank + r
         new = lambda *shape: torch.empty(shape, dtype=x.dtype, device=x.device)  # noqa: E731
-        rope = self.rope
-        freq, rot_dims, mult = (rope.freq, rope.dims, rope.mult) if rope is not None else (None, 0, 1.0)
+        turns = self._turns(ctx)
         proj = ops.linear(x, self.params["proj.weight"], None, out_dtype=torch.float32)
         ld = proj.shape[1]
         q = proj
@@ -131,14 +140,13 @@ class LatentAttention(Mixer):
             query = (0, self.params["q_down_norm.weight"], latent_q)
         writes = self.own_keys and cache.writes
         if writes or query is not None:
-            ops.latent_prepare(proj, cache.pages, ctx.slot_mappings[cache.group] if writes else None, ctx.positions,
-                               self.down_offset, rank, r, self.p("down_norm.weight"), self.norm_eps, freq, rot_dims, mult,
-                               query)
+            ops.latent_prepare(proj, cache.pages, ctx.slot_mappings[cache.group] if writes else None, self.down_offset,
+                               rank, r, self.p("down_norm.weight"), self.norm_eps, turns, query)
         if query is not None:
             q = ops.linear(latent_q, self.params["q_up.weight"], None, out_dtype=torch.float32)
         q_abs = new(T, H, width)
         ops.heads_gemm(q, 0, q.shape[1], d + r, self.up_k, q_abs, 0, H * width, width, H, T, rank, d, alpha=self.scale,
-                       turn=QueryTurn(d, rank, r, rot_dims, freq, mult, self.scale, ctx.positions))
+                       turn=QueryTurn(d, rank, r, turns, self.scale))
         latent = new(T, H, rank)
         ops.latent_attention(q_abs, cache.pages, latent, self._meta(ctx, cache.group), rank, self.p("sink"), self.window)
         out = new(T, H * dv)

@@ -68,6 +68,11 @@ class ScaledRotary(PositionEncoding):
         self.freq: torch.Tensor | None = None
         self.mult = 1.0
 
+    @property
+    def identity(self) -> tuple:
+        """Equal for rotations that turn alike."""
+        return (type(self).__name__, self.dims, self.base, self.scaling)
+
     def frequencies(self) -> tuple[torch.Tensor, float]:
         i = torch.arange(self.dims // 2, dtype=torch.float64)
         f = self.base ** (-2.0 * i / max(self.dims, 1))

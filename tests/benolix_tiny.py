@@ -94,8 +94,20 @@ BENO_D = {
     ),
 }
 
-CONFIGS = {"A": BENO_A, "B": BENO_B, "C": BENO_C, "D": BENO_D}
-SEEDS = {"A": 5, "B": 15, "C": 25, "D": 45}
+# E: latents and experts of sizes that the tile kernels for real models take
+BENO_E = {
+    "architecture": "Benolix", "vocab": 101, "width": 128, "embedding": {"scale": 3.0}, "norm": {"eps": 1e-5},
+    "postln_alpha": 1.7,
+    "layers": _layers(
+        (_attn(5, 40, 64, 24, 128, 72, 70), _moe(64, 3, 2, identity=1, limit=1.8, scale=1.5)),
+        (_attn(16, 16, 64, 8, 128, 48, 131, kv_from=0), _dense(192)),
+        (_attn(20, 24, 64, 16, 256, 96, None, base=3000.0), _moe(128, 2, 1, identity=2, limit=0.9, scale=0.8)),
+        (_attn(2, 32, 64, 64, 256, 56, 65, base=3000.0, kv_from=2), None),
+    ),
+}
+
+CONFIGS = {"A": BENO_A, "B": BENO_B, "C": BENO_C, "D": BENO_D, "E": BENO_E}
+SEEDS = {"A": 5, "B": 15, "C": 25, "D": 45, "E": 65}
 BARE_SECOND_NORM = {("D", 1)}     # layers without feed-forward whose checkpoint holds a second norm all the same
 
 

@@ -267,30 +267,32 @@ class PlainKernels:
     def linear_f32(self, x, weight, bias=None):
         return self.linear(x, weight, bias, out_dtype=torch.float32)
 
-    @staticmethod
-    def _turn(x, positions, freq, rot_dims, mult):
-        """x [T, ..., n]: neighbouring pairs of the first ``rot_dims`` entries turned by position * freq."""
-        if not rot_dims:
-            return x
+    def rotation_table(self, positions, freq, mult=1.0):
         ang = positions.to(WIDE)[:, None] * freq.to(WIDE)[None, :]
-        c, s_ = torch.cos(ang) * mult, torch.sin(ang) * mult
+        return torch.stack((torch.cos(ang) * mult, torch.sin(ang) * mult), dim=-1).to(torch.float32)
+
+    @staticmethod
+    def _turn(x, turns):
+        """x [T, ..., n]: neighbouring pairs of its first entries turned by the table's cosines and sines."""
+        if turns is None:
+            return x
+        c, s_, dims = turns[..., 0].to(WIDE), turns[..., 1].to(WIDE), 2 * turns.shape[1]
         while c.dim() < x.dim():
             c, s_ = c.unsqueeze(1), s_.unsqueeze(1)
         out = x.clone()
-        u, v = x[..., 0:rot_dims:2], x[..., 1:rot_dims:2]
-        out[..., 0:rot_dims:2] = u * c - v * s_
-        out[..., 1:rot_dims:2] = v * c + u * s_
+        u, v = x[..., 0:dims:2], x[..., 1:dims:2]
+        out[..., 0:dims:2] = u * c - v * s_
+        out[..., 1:dims:2] = v * c + u * s_
         return out
 
-    def latent_prepare(self, proj, pages, slots, positions, kv_off, rank, rot, norm_weight, eps, freq=None, rot_dims=0,
-                       mult=1.0, query=None):
+    def latent_prepare(self, proj, pages, slots, kv_off, rank, rot, norm_weight, eps, turns=None, query=None):
         p = proj.to(WIDE)
         if query is not None:
             off, weight, out = query
             out.copy_((pl.rms_unit(p[:, off:off + out.shape[1]], eps) * weight.to(WIDE)).to(out.dtype))
         if slots is not None:
             c = pl.rms_unit(p[:, kv_off:kv_off + rank], eps) * norm_weight.to(WIDE)
-            k = self._turn(p[:, kv_off + rank:kv_off + rank + rot], positions, freq, rot_dims, mult)
+            k = self._turn(p[:, kv_off + rank:kv_off + rank + rot], turns)
             flat = pages.view(-1, rank + rot)
             for t in range(proj.shape[0]):
                 if int(slots[t]) >= 0:
@@ -310,7 +312,7 @@ class PlainKernels:
             torch.as_strided(yf, (m, n), (ldy, 1), y_offset + h * hsy).copy_(r.to(y.dtype))
             if turn is not None and turn.rot:
                 part = torch.as_strided(xf, (m, turn.rot), (ldx, 1), turn.x_offset + h * hsx).to(WIDE)
-                part = self._turn(part, turn.positions, turn.freq, turn.rot_dims, turn.mult) * turn.scale
+                part = self._turn(part, turn.turns) * turn.scale
                 torch.as_strided(yf, (m, turn.rot), (ldy, 1), turn.y_offset + h * hsy).copy_(part.to(y.dtype))
         return y
 

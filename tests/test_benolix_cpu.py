@@ -20,7 +20,7 @@ from atom_amd.models.model import LayerRun
 from atom_amd.parts.base import KVCacheNeed, LatentCacheNeed, StateNeed
 from atom_amd.weights.loader import expected_tensors
 
-LENGTHS = {"A": [1, 7, 33, 70], "B": [2, 19, 45, 64], "C": [3, 52], "D": [1, 2, 30, 41]}
+LENGTHS = {"A": [1, 7, 33, 70], "B": [2, 19, 45, 64], "C": [3, 52], "D": [1, 2, 30, 41], "E": [2, 45]}
 WHICH = sorted(LENGTHS)
 
 
@@ -78,7 +78,7 @@ def test_plain_mechanisms_show():
 
 
 @pytest.mark.parametrize("which,layer", [("A", 0), ("A", 1), ("A", 3), ("B", 0), ("B", 1), ("B", 2), ("B", 3), ("C", 0),
-                                         ("C", 1), ("C", 2), ("D", 2)])
+                                         ("C", 1), ("C", 2), ("D", 2), ("E", 0), ("E", 1), ("E", 3)])
 @pytest.mark.parametrize("off", [-1, 1])
 def test_plain_a_window_one_token_off_shows(which, layer, off):
     """With these weights a window that is one token off is seen, from the first position it can matter at."""

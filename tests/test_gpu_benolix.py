@@ -62,18 +62,20 @@ def test_query_latent_and_key_rows(dtype, cq, rank, rot, dims):
     for t in range(T):
         if slots[t] >= 0:
             want[slots[t]] = keys[t]
-    freq = frequencies(dims, 777.0) if dims else None
-    dev, dpos, dslots = proj.to(DEV), positions.int().to(DEV), slots.int().to(DEV)
+    turns = ops.rotation_table(positions.int().to(DEV), frequencies(dims, 777.0)) if dims else None
+    dev, dslots = proj.to(DEV), slots.int().to(DEV)
     for with_query, with_keys in ((True, True), (True, False), (False, True)):
         out = torch.zeros((T, cq), dtype=dtype, device=DEV)
         pages = torch.zeros((3, 4, rank + rot), dtype=dtype, device=DEV)
-        ops.latent_prepare(dev, pages, dslots if with_keys else None, dpos, off, rank, rot,
-                           wk.to(DEV) if with_keys else None, eps, freq, dims, 1.0,
-                           (pre, wq.to(DEV), out) if with_query else None)
+        ops.latent_prepare(dev, pages, dslots if with_keys else None, off, rank, rot, wk.to(DEV) if with_keys else None, eps,
+                           turns, (pre, wq.to(DEV), out) if with_query else None)
         close(out, want_q if with_query else 0 * want_q, dtype, "query latent")
         close(pages.view(12, -1), want if with_keys else 0 * want, dtype, "pages")
     with pytest.raises(KernelError):
-        ops.latent_prepare(dev, pages, dslots, dpos, proj.shape[1] - 3, rank, rot, wk.to(DEV), eps, freq, dims, 1.0, None)
+        ops.latent_prepare(dev, pages, dslots, proj.shape[1] - 3, rank, rot, wk.to(DEV), eps, turns)
+    if dims:
+        with pytest.raises(KernelError):
+            ops.latent_prepare(dev, pages, dslots, off, rank, dims - 2, wk.to(DEV), eps, turns)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -112,9 +114,9 @@ def test_absorbing_product_turns_the_rotated_parts(dtype, H, m, d, rot, dims, ra
     up = rnd((H, rank, d), 2, d ** -0.5).to(dtype)
     positions = torch.randint(0, 60000, (m,), generator=torch.Generator().manual_seed(3))
     out = torch.zeros((m, H, width), dtype=dtype, device=DEV)
-    freq = frequencies(dims, 5e5) if dims else None
+    turns = ops.rotation_table(positions.int().to(DEV), frequencies(dims, 5e5)) if dims else None
     ops.heads_gemm(q.to(DEV), 0, ld, d + rot, up.to(DEV), out, 0, H * width, width, H, m, rank, d, alpha=0.3,
-                   turn=QueryTurn(d, rank, rot, dims, freq, 1.0, 0.3, positions.int().to(DEV)))
+                   turn=QueryTurn(d, rank, rot, turns, 0.3))
     heads = q.double().view(m, H, d + rot)
     close(out[..., :rank], torch.stack([heads[:, h, :d] @ up[h].double().T for h in range(H)], 1) * 0.3, dtype, "absorbed")
     close(out[..., rank:], pb.rotate_neighbours(heads[..., d:], positions, dims, 5e5) * 0.3, dtype, "turned")
@@ -275,7 +277,7 @@ def test_experts_with_clamped_gates_and_identities(dtype, width, ff, experts, id
 
 # ------------------------------------------------------------------ the engine
 
-LENGTHS = {"A": [1, 7, 33, 150, 64, 300], "B": [2, 19, 45, 260, 128], "C": [3, 40, 17, 200, 140], "D": [1, 2, 40, 130, 33]}
+LENGTHS = {"A": [1, 7, 33, 150, 64, 300], "B": [2, 19, 45, 260, 128], "C": [3, 40, 17, 200, 140], "D": [1, 2, 40, 130, 33], "E": [2, 33, 310, 200, 17]}
 WHICH = sorted(LENGTHS)
 # float32: every position, against the largest logit of its request.  bfloat16: an expert chosen by a hair may be
 # another one after rounding, which changes that token and, through its cached latents, later ones a little; so tokens
@@ -332,7 +334,7 @@ def test_cuts_match_plain(which, cut, dtype):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("which", ["A", "C"])
+@pytest.mark.parametrize("which", ["A", "C", "E"])
 def test_small_pages_slots_used_again_and_long_decoding(which, dtype):
     """Pages of 4 tokens, two state slots for five requests, and 200 tokens decoded one by one past every window, each of
     them compared."""
@@ -345,7 +347,7 @@ def test_small_pages_slots_used_again_and_long_decoding(which, dtype):
     _check(steps, results, requests, which, dtype, f"{which}/page4/{dtype}")
 
 
-@pytest.mark.parametrize("which", ["A", "B"])
+@pytest.mark.parametrize("which", ["A", "B", "E"])
 def test_logits_do_not_depend_on_the_batch_or_the_cut(which):
     """float32: a request's logits alone, cut in portions, and beside others differ by rounding of sums only."""
     requests = _requests(which)
@@ -386,7 +388,7 @@ def test_stream_after_every_layer(which):
         close(mine, want, torch.float32, f"after layer {layer}")
 
 
-@pytest.mark.parametrize("which,dtype", [("A", "fp32"), ("B", "fp32"), ("C", "fp32"), ("D", "fp32"), ("B", "bf16")])
+@pytest.mark.parametrize("which,dtype", [("A", "fp32"), ("B", "fp32"), ("C", "fp32"), ("D", "fp32"), ("B", "bf16"), ("E", "bf16")])
 def test_greedy_generation_through_the_engine(which, dtype):
     from atom_amd import LLMEngine, SamplingParams
 

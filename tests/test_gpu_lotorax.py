@@ -121,13 +121,14 @@ def test_latent_prepare(dtype, heads, dim, rot, rank, dims, scaling):
     q_abs = torch.zeros((T, heads, rank + rot), dtype=dtype, device=DEV)
     kv_off = pre + heads * (dim + rot)
     where, dpos = proj.to(DEV), positions.int().to(DEV)
-    ops.latent_prepare(where, pages, slots.int().to(DEV), dpos, kv_off, rank, rot, w.to(DEV), 1e-5, rope.freq, dims, rope.mult)
+    turns = ops.rotation_table(dpos, rope.freq, rope.mult)
+    ops.latent_prepare(where, pages, slots.int().to(DEV), kv_off, rank, rot, w.to(DEV), 1e-5, turns)
     # the queries' rotated parts go past the absorbing product, whatever kernel takes it
     up = rnd((heads, rank, dim), 3, dim ** -0.5).to(dtype).to(DEV)
     for rows in (T, 3):
         q_abs.zero_()
         ops.heads_gemm(where, pre, ld, dim + rot, up, q_abs, 0, heads * (rank + rot), rank + rot, heads, rows, rank, dim,
-                       alpha=0.37, turn=QueryTurn(pre + dim, rank, rot, dims, rope.freq, rope.mult, 0.37, dpos[:rows]))
+                       alpha=0.37, turn=QueryTurn(pre + dim, rank, rot, turns[:rows].contiguous(), 0.37))
         p = proj.double()[:rows]
         q = p[:, pre:kv_off].view(rows, heads, dim + rot)
         close(q_abs[:rows, :, rank:], pl.rotate_pairs(q[..., dim:], positions[:rows], dims, 5000.0, scaling) * 0.37, dtype,
